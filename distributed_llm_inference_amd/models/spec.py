@@ -91,10 +91,20 @@ class LayerSpec:
     matrix before mask and softmax, s_h <- sum_g M[h, g] s_g. `chunk` > 0: a query at i sees the keys j <= i of its own
     chunk only, floor(i / chunk) = floor(j / chunk), chunks counted from the sequence's position 0.
     ``parallel`` with `branch_scales` (a, b): the branches' outputs are added as a * left + b * right (no norms, no average).
+    ``linear_attention``: a recurrence without softmax or denominator per head over a [dim, vdim] state,
+    S <- diag(a) S + k v^T, o = S^T q, with a decay `head_decay` per head from the config, or (no `head_decay`) one per key
+    channel, sigmoid(z)^(1 / `tau`) with z a projection of low rank `rank` plus a bias. `scale` multiplies the scores (q . k);
+    the read-out is RMS-normed over each head's values (with a weight shared by the heads when `o_norm`), multiplied by
+    silu(W_g h) and projected.
+    ``latent_attention`` without a query latent (`q_rank` 0) projects its queries from the mixer's input directly; `window`
+    limits it as above; `kv_from` = j >= 0: the layer keeps nothing of its own and reads layer j's latents and rotated key
+    parts (its own query, key and value projections, window and scale).
     The feed-forward sublayer is `ff_kind`: ``gated_gelu`` (gelu_tanh(gate) * up, biases), ``gelu`` (up, exact
     GELU, down; no biases), ``xielu`` (up, a two-sided quadratic / exponential unit with two learned numbers, down),
-    ``relu2`` (up, the square of relu, down; biases) or ``moe`` (`moe` says how tokens are routed to its experts)."""
-    kind: str                       # "attention" | "delta" | "general_delta" | "mlstm" | "parallel" | "rglru" | "latent_attention"
+    ``relu2`` (up, the square of relu, down; biases), ``polynorm`` (up, a N(z) + b N(z^2) + c N(z^3) + e with four learned
+    numbers, N dividing a token's row by its root mean square, down) or ``moe`` (`moe` says how tokens are routed to its experts)."""
+    # "attention" | "delta" | "general_delta" | "mlstm" | "parallel" | "rglru" | "latent_attention" | "linear_attention"
+    kind: str
     heads: int
     kv_heads: int
     dim: int
@@ -136,6 +146,10 @@ class LayerSpec:
     head_mix: bool = False
     chunk: int = 0
     branch_scales: tuple = ()
+    head_decay: tuple = ()
+    tau: float = 1.0
+    o_norm: bool = False
+    kv_from: int = -1
 
     @property
     def group(self) -> int:
@@ -144,7 +158,7 @@ class LayerSpec:
     @property
     def has_state(self) -> bool:
         """The mixer keeps a per-sequence state in the sequence's slot."""
-        return self.kind in ("delta", "general_delta", "mlstm", "rglru") or any(b.has_state for b in self.branches)
+        return self.kind in ("delta", "general_delta", "mlstm", "rglru", "linear_attention") or any(b.has_state for b in self.branches)
 
     @property
     def has_ff(self) -> bool:
@@ -163,6 +177,13 @@ class LayerSpec:
         if self.kind == "rglru":
             w = self.rec_width
             return 3 * w * width + 2 * w * (w // self.blocks) + w * (self.conv + 6)
+        if self.kind == "linear_attention":
+            n = width * self.heads * (2 * self.dim + 3 * self.vdim) + (self.vdim if self.o_norm else 0)
+            return n if self.head_decay else n + (self.rank or 16) * (width + self.heads * self.dim) + self.heads * self.dim
+        if self.kind == "latent_attention" and not self.q_rank:
+            kept = width * (self.kv_rank + self.rot_dim) + self.kv_rank if self.kv_from < 0 else 0
+            return width * self.heads * (self.dim + self.rot_dim) + kept + self.kv_rank * self.heads * (self.dim + self.vdim) \
+                + self.heads * self.vdim * width
         if self.kind == "latent_attention":
             return width * (self.q_rank + self.kv_rank + self.rot_dim) + self.q_rank * self.heads * (self.dim + self.rot_dim) \
                 + self.kv_rank * self.heads * (self.dim + self.vdim) + self.heads * self.vdim * width + self.q_rank + self.kv_rank
@@ -185,7 +206,7 @@ class LayerSpec:
     def ff_param_count(self, width: int) -> int:
         if self.moe is not None:
             return self.moe.experts * (3 * width * self.moe.ff + width) + 3 * width * self.moe.shared_ff
-        if self.ff_kind in ("gelu", "xielu"):
+        if self.ff_kind in ("gelu", "xielu", "polynorm"):
             return 2 * width * self.ff
         if self.ff_kind == "relu2":
             return 2 * width * self.ff + self.ff + width
@@ -205,8 +226,10 @@ class MoeSpec:
     `group_rank`: how many of a block's best choice scores are added up to rank it (1: its best). `renorm` off: the weights
     are the chosen scores times `scale`, not divided by their sum. `identity`: the router has that many outputs more than
     there are experts; choosing one of them returns the token's input itself (times the weight); they count as experts for
-    the groups. `shared_ff` > 0: one more expert of that width runs for every token and is added unweighted. `act`
-    ``silu``: an expert computes down(silu(gate(x)) * up(x)), no limits."""
+    the groups. `shared_ff` > 0: one more expert of that width runs for every token and is added unweighted, or (`shared_gate`)
+    multiplied by the sigmoid of one more projection of the token to a single number; `shared_limit` is its activation's limit.
+    `act` ``silu``: an expert computes down(silu(gate(x)) * up(x)), no limits. `score` ``table``: there is no router; a table
+    [vocab, top] of expert numbers names each token's experts by the token's id, each weighted 1 / top."""
     experts: int
     top: int
     ff: int
@@ -221,6 +244,8 @@ class MoeSpec:
     identity: int = 0
     shared_ff: int = 0
     act: str = "swish_lim"
+    shared_gate: bool = False
+    shared_limit: float = 0.0
 
     @property
     def outputs(self) -> int:
@@ -231,7 +256,7 @@ class MoeSpec:
 @dataclass(frozen=True)
 class ModelSpec:
     name: str
-    family: str                     # "llama" | "gpt2" | "letarax" | "nufapel" | "tezesun" | "zovozen"
+    family: str                     # "llama" | "gpt2" | "letarax" | "nufapel" | "tezesun" | "zovozen" | "pifutar"
     num_layers: int
     hidden_size: int
     num_heads: int
@@ -279,6 +304,11 @@ class ModelSpec:
     # `post_norm`: the sublayers read the residual stream itself and a plain-weight RMS norm sits on their OUTPUT only:
     # x += norm1(mixer(x)); x += norm2(ff(x))
     post_norm: bool = False
+    # `input_conv` > 0: what every sublayer reads is h + a causal convolution of h over that many tokens, per channel (h the
+    # sublayer's normed input; the last input_conv - 1 of them are per-sequence state of every sublayer). `depth_average`:
+    # what goes on from a layer is a learned weighted sum of the embedding and of all layers' results so far
+    input_conv: int = 0
+    depth_average: bool = False
 
     @property
     def is_hybrid(self) -> bool:
@@ -288,7 +318,7 @@ class ModelSpec:
     def has_recurrent_state(self) -> bool:
         """Some layer keeps a per-sequence state that lives in the sequence's slot (not in cache blocks): a sequence
         cannot change slots without its state being moved along."""
-        return self.token_shift or any(l.has_state for l in self.layer_specs)
+        return self.token_shift or self.input_conv > 1 or any(l.has_state for l in self.layer_specs)
 
     def layer_runs(self):
         """[(layer, pass)] in the order the layers run; pass is -1 outside the repeated stretch, else the number of the
@@ -592,6 +622,96 @@ class ModelSpec:
             bos_token_id=cfg.get("bos_token_id"), eos_token_id=_scalar_eos(cfg.get("eos_token_id")), hf_type="zovozen",
             layer_specs=tuple(layers), post_norm=True)
 
+    @staticmethod
+    def from_pifutar_config(cfg: Dict[str, Any], name: str = "") -> "ModelSpec":
+        """Pifutar: pre-norm layers whose sublayers read their normed input plus a short causal convolution of it
+        (``canon.taps``), with a learned average over depth behind every layer. ``layers`` lists for each layer its ``type`` —
+        ``gla`` (mixer: heads, dim, vdim, tau: decays per key channel), ``retention`` (heads, dim, vdim, decay: one number
+        per head) or ``latent_attention`` (heads, dim, rot_dim, vdim, kv_rank, scale, mask.size = window, rot.dims / base,
+        kv_from = the layer whose latents are read) — and its ``mlp``: null, ``dense`` (ff) or ``moe`` (expert.ff / limit,
+        router.experts / top, shared.ff / limit; experts by a table over token ids). The head is the embedding table. Keys a
+        config leaves out switch their mechanism off."""
+        layers = []
+        for i, l in enumerate(cfg["layers"]):
+            m, mlp = l["mixer"], l.get("mlp")
+            ffkw: Dict[str, Any] = dict(ff=0, ff_kind="polynorm")
+            if mlp is not None and mlp.get("kind", "dense") == "dense":
+                ffkw = dict(ff=int(mlp["ff"]), ff_kind="polynorm")
+            elif mlp is not None and mlp["kind"] == "moe":
+                r, e, sh = mlp["router"], mlp["expert"], mlp.get("shared") or {}
+                moe = MoeSpec(experts=int(r["experts"]), top=int(r["top"]), ff=int(e["ff"]), limit=float(e["limit"]), score="table",
+                              renorm=False, shared_ff=int(sh.get("ff") or 0), shared_gate=bool(sh.get("ff")),
+                              shared_limit=float(sh.get("limit", e["limit"])))
+                if not 1 <= moe.top <= moe.experts:
+                    raise ValueError(f"layer {i}: {moe.experts} experts, {moe.top} chosen")
+                ffkw = dict(ff=0, ff_kind="moe", moe=moe)
+            elif mlp is not None:
+                raise ValueError(f"layer {i}: feed-forward kind {mlp.get('kind')!r} is not supported (dense and moe are)")
+            H, d, dv = int(m["heads"]), int(m["dim"]), int(m["vdim"])
+            if l["type"] in ("gla", "retention"):
+                kw: Dict[str, Any] = dict(head_decay=tuple(float(x) for x in m["decay"])) if l["type"] == "retention" else \
+                    dict(tau=float(m["tau"]), rank=int(m.get("rank", 0)), o_norm=True)
+                if l["type"] == "retention" and len(kw["head_decay"]) != H:
+                    raise ValueError(f"layer {i}: {len(kw['head_decay'])} decays for {H} heads")
+                layers.append(LayerSpec("linear_attention", heads=H, kv_heads=H, dim=d, vdim=dv, scale=d ** -0.5, **kw, **ffkw))
+            elif l["type"] == "latent_attention":
+                rot, dr, src = m.get("rot") or {}, int(m["rot_dim"]), m.get("kv_from")
+                rd = int(rot.get("dims") or 0)
+                if rd % 2 or rd > dr:
+                    raise ValueError(f"layer {i}: {rd} rotated entries in a part of {dr}")
+                win = (m.get("mask") or {}).get("size")
+                layers.append(LayerSpec("latent_attention", heads=H, kv_heads=1, dim=d, vdim=dv, scale=float(m["scale"]), kv_rank=int(m["kv_rank"]),
+                                        rot_dim=dr, window=int(win) if win else None, rope_dims=rd, rope_base=float(rot.get("base", 10000.0)),
+                                        rope_interleaved=True, kv_from=-1 if src is None else int(src), **ffkw))
+                if src is not None:
+                    j = layers[int(src)] if 0 <= int(src) < i else None
+                    a = layers[-1]
+                    if j is None or j.kind != "latent_attention" or j.kv_from >= 0 or (j.kv_rank, j.rot_dim, j.rope_dims, j.rope_base) != \
+                            (a.kv_rank, a.rot_dim, a.rope_dims, a.rope_base):
+                        raise ValueError(f"layer {i} reads the latents of layer {src}, which keeps none of the same sizes and rotation")
+            else:
+                raise ValueError(f"layer {i}: unknown mixer type {l['type']!r}")
+        if not layers:
+            raise ValueError("a model needs at least one layer")
+        att = [l for l in layers if l.kind == "latent_attention"] or layers
+        return ModelSpec(
+            name=name or "pifutar", family="pifutar", num_layers=len(layers), hidden_size=int(cfg["width"]),
+            num_heads=max(l.heads for l in att), num_kv_heads=max(l.kv_heads for l in att), head_dim=max(max(l.dim, l.vdim) for l in att),
+            intermediate_size=max(max(l.ff, l.moe.ff if l.moe else 0, l.moe.shared_ff if l.moe else 0) for l in layers),
+            vocab_size=int(cfg["vocab"]), max_position=1 << 30, norm_eps=float(cfg["norm"]["eps"]), tie_embeddings=True,
+            bos_token_id=cfg.get("bos_token_id"), eos_token_id=_scalar_eos(cfg.get("eos_token_id")), hf_type="pifutar",
+            layer_specs=tuple(layers), input_conv=int((cfg.get("canon") or {}).get("taps") or 0), depth_average=True)
+
+    def pifutar_config(self) -> Dict[str, Any]:
+        """The inverse of `from_pifutar_config` (`rank` is a size a checkpoint's tensors give; it is written so that random
+        weights of the same shapes can be drawn from the config alone)."""
+        out = []
+        for l in self.layer_specs:
+            m: Dict[str, Any] = {"heads": l.heads, "dim": l.dim, "vdim": l.vdim}
+            kind = l.kind
+            if kind == "linear_attention":
+                kind = "retention" if l.head_decay else "gla"
+                m.update({"decay": list(l.head_decay)} if l.head_decay else {"tau": l.tau, "rank": l.rank})
+            else:
+                m.update({"rot_dim": l.rot_dim, "kv_rank": l.kv_rank, "scale": l.scale})
+                if l.rope_dims:
+                    m["rot"] = {"base": l.rope_base, "dims": l.rope_dims}
+                if l.window:
+                    m["mask"] = {"size": l.window}
+                if l.kv_from >= 0:
+                    m["kv_from"] = l.kv_from
+            if l.moe is not None:
+                e = l.moe
+                mlp: Optional[Dict[str, Any]] = {"kind": "moe", "expert": {"ff": e.ff, "limit": e.limit},
+                                                 "router": {"experts": e.experts, "top": e.top}}
+                if e.shared_ff:
+                    mlp["shared"] = {"ff": e.shared_ff, "limit": e.shared_limit}
+            else:
+                mlp = {"kind": "dense", "ff": l.ff} if l.ff else None
+            out.append({"type": kind, "mixer": m, "mlp": mlp})
+        return {"architecture": "Pifutar", "layers": out, "canon": {"taps": self.input_conv}, "norm": {"eps": self.norm_eps},
+                "vocab": self.vocab_size, "width": self.hidden_size, "bos_token_id": self.bos_token_id, "eos_token_id": self.eos_token_id}
+
     def zovozen_config(self) -> Dict[str, Any]:
         """The inverse of `from_zovozen_config`."""
         out = []
@@ -703,6 +823,8 @@ class ModelSpec:
             return ModelSpec.from_tezesun_config(cfg, name=name)
         if cfg.get("architecture") == "Zovozen":
             return ModelSpec.from_zovozen_config(cfg, name=name)
+        if cfg.get("architecture") == "Pifutar":
+            return ModelSpec.from_pifutar_config(cfg, name=name)
         if mt == "gpt2" or any("GPT2" in a for a in archs):
             if cfg.get("activation_function", "gelu_new") != "gelu_new" or cfg.get("scale_attn_by_inverse_layer_idx"):
                 raise ValueError("GPT-2 variants other than gelu_new MLPs with plain 1/sqrt(d) attention scaling are not supported")
@@ -834,7 +956,8 @@ class ModelSpec:
     def hf_config(self) -> Dict[str, Any]:
         """The inverse of `from_hf_config`: a config.json dict for this spec."""
         if self.is_hybrid:
-            return {"nufapel": self.nufapel_config, "tezesun": self.tezesun_config, "zovozen": self.zovozen_config}.get(self.family, self.letarax_config)()
+            return {"nufapel": self.nufapel_config, "tezesun": self.tezesun_config, "zovozen": self.zovozen_config,
+                    "pifutar": self.pifutar_config}.get(self.family, self.letarax_config)()
         if self.is_gpt2:
             return {
                 "model_type": "gpt2", "architectures": ["GPT2LMHeadModel"],
@@ -1034,6 +1157,35 @@ def zovozen_spec(name: str, width: int, heads: int, kv_heads: int, head_dim: int
                      tie_embeddings=True, bos_token_id=1, eos_token_id=2, hf_type="zovozen", layer_specs=layers, post_norm=True)
 
 
+def pifutar_spec(name: str, width: int, heads: int, head_dim: int, ff: int, num_layers: int, window: int, vocab_size: int = 32000,
+                 pattern: str = "rgls", experts: int = 8, top: int = 2, kv_rank: int = 0, rot_dim: int = 0, vdim: int = 0, rank: int = 16,
+                 taps: int = 4, dense: str = "d---") -> ModelSpec:
+    """A Pifutar stack from a few numbers: `pattern` repeats over the layers ('r' retention, 'g' gated linear attention, 'l'
+    latent attention with a window, 's' latent attention that reads the latents of the last 'l' layer before it); `dense` repeats
+    over the layers' feed-forwards: 'd' dense of `ff`, 'n' none, else routed by token id (`experts` experts of ff / 4, `top` per
+    token, a gated shared expert of ff / 2)."""
+    dv, dr = vdim or head_dim, rot_dim or max(2, head_dim // 2)
+    moe = MoeSpec(experts=experts, top=top, ff=max(8, ff // 4), limit=7.0, score="table", renorm=False, shared_ff=max(8, ff // 2), shared_gate=True,
+                  shared_limit=7.0)
+    decay = tuple(1.0 - 2.0 ** -(5.0 + 3.0 * i / max(1, heads - 1)) for i in range(heads))
+    layers, last = [], -1
+    for i in range(num_layers):
+        c, f = pattern[i % len(pattern)], dense[i % len(dense)]
+        kw: Dict[str, Any] = dict(ff=ff, ff_kind="polynorm") if f == "d" else dict(ff=0, ff_kind="polynorm") if f == "n" else dict(ff=0, ff_kind="moe", moe=moe)
+        if c in "rg":
+            kw.update(head_decay=decay) if c == "r" else kw.update(tau=16.0, rank=rank, o_norm=True)
+            layers.append(LayerSpec("linear_attention", heads=heads, kv_heads=heads, dim=head_dim, vdim=dv, scale=head_dim ** -0.5, **kw))
+        else:
+            src = last if c == "s" else -1
+            last = i if src < 0 else last
+            layers.append(LayerSpec("latent_attention", heads=heads, kv_heads=1, dim=head_dim, vdim=dv, scale=(head_dim + dr) ** -0.5, window=window,
+                                    kv_rank=kv_rank or max(8, width // 8), rot_dim=dr, rope_dims=dr, rope_base=500000.0, rope_interleaved=True,
+                                    kv_from=src, **kw))
+    return ModelSpec(name=name, family="pifutar", num_layers=num_layers, hidden_size=width, num_heads=heads, num_kv_heads=1, head_dim=max(head_dim, dv),
+                     intermediate_size=ff, vocab_size=vocab_size, max_position=1 << 30, norm_eps=1e-5, tie_embeddings=True, bos_token_id=1,
+                     eos_token_id=2, hf_type="pifutar", layer_specs=tuple(layers), input_conv=taps, depth_average=True)
+
+
 # Letarax stacks of the sizes of the Llama benchmark shapes (random weights; `bench.py --hybrid-compare` runs them)
 BUILTIN_SPECS["letarax-1b-like"] = letarax_spec("letarax-1b-like", 2048, 16, 4, 128, 8192, 8, 1024)
 BUILTIN_SPECS["letarax-8b-like"] = letarax_spec("letarax-8b-like", 4096, 32, 8, 128, 14336, 4, 2048)
@@ -1046,6 +1198,9 @@ BUILTIN_SPECS["tezesun-8b-like"] = tezesun_spec("tezesun-8b-like", 4096, 32, 8, 
 # Zovozen stacks of the same sizes (`bench.py --postnorm-compare` runs them beside the Nufapel stacks)
 BUILTIN_SPECS["zovozen-1b-like"] = zovozen_spec("zovozen-1b-like", 2048, 16, 4, 128, 8192, 8, chunk=1024)
 BUILTIN_SPECS["zovozen-8b-like"] = zovozen_spec("zovozen-8b-like", 4096, 32, 8, 128, 14336, 4, chunk=2048)
+# Pifutar stacks of the same sizes (`bench.py --canon-compare` runs them beside the Tezesun and Nufapel stacks)
+BUILTIN_SPECS["pifutar-1b-like"] = pifutar_spec("pifutar-1b-like", 2048, 16, 128, 8192, 8, window=1024, kv_rank=448, rot_dim=64)
+BUILTIN_SPECS["pifutar-8b-like"] = pifutar_spec("pifutar-8b-like", 4096, 32, 128, 14336, 4, window=2048, kv_rank=448, rot_dim=64)
 
 
 def _register_test_models():
@@ -1073,6 +1228,10 @@ def _register_test_models():
                                                       identity=2, groups=4, keep=2, chunk=20, vdim=24, rot_dims=8)
     BUILTIN_SPECS["tiny-zovozen-gpu-test"] = zovozen_spec("tiny-zovozen-gpu-test", 128, 4, 2, 32, 256, 4, vocab_size=320, pattern="mdm",
                                                           experts=6, identity=2, groups=2, keep=1, chunk=40, vdim=48, rot_dims=16)
+    BUILTIN_SPECS["tiny-pifutar-test"] = pifutar_spec("tiny-pifutar-test", 64, 4, 16, 96, 5, window=12, vocab_size=320, pattern="lgrsl", experts=5,
+                                                      kv_rank=20, rot_dim=8, vdim=24, rank=4, taps=3, dense="-d-n-")
+    BUILTIN_SPECS["tiny-pifutar-gpu-test"] = pifutar_spec("tiny-pifutar-gpu-test", 128, 4, 32, 256, 5, window=36, vocab_size=320, pattern="rglsg",
+                                                          experts=6, kv_rank=40, rot_dim=16, vdim=48, rank=8, taps=4, dense="d--")
     BUILTIN_SPECS["tiny-gpt2-gpu-test"] = tiny_spec(
         "gpt2", name="tiny-gpt2-gpu-test", hidden_size=256, num_heads=4, num_kv_heads=4, head_dim=64,
         intermediate_size=1024, vocab_size=333, num_layers=4)

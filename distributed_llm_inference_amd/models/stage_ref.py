@@ -62,6 +62,9 @@ class RefStage:
                 if self.spec.token_shift:           # every layer also carries the previous token's normed input
                     for st in c:
                         st.append(torch.zeros(self.spec.hidden_size, dtype=torch.float32, device=self.device))
+                if self.spec.input_conv:            # every sublayer also carries its convolution's last inputs
+                    for st in c:
+                        st += [torch.zeros(self.spec.input_conv - 1, self.spec.hidden_size, dtype=torch.float32, device=self.device) for _ in range(2)]
             else:
                 z = lambda: torch.zeros(0, self.spec.num_kv_heads, self.spec.head_dim, dtype=self.dtype, device=self.device)
                 c = [[z(), z()] for _ in self.plan.layers]
@@ -79,6 +82,8 @@ class RefStage:
             return [z32(ls.heads, ls.dim, ls.vdim), z32(ls.heads, ls.dim), z32(ls.heads)]
         if ls.kind == "rglru":
             return [z32(max(ls.conv - 1, 0), ls.rec_width), z32(ls.rec_width)]
+        if ls.kind == "linear_attention":
+            return [z32(ls.heads, ls.dim, ls.vdim)]
         if ls.kind == "latent_attention":
             return [torch.zeros(0, 1, ls.kv_rank, dtype=self.dtype, device=dev), torch.zeros(0, 1, ls.rot_dim, dtype=self.dtype, device=dev)]
         if ls.kind == "attention":
@@ -429,10 +434,123 @@ class RefStage:
             self.layer_outputs.append(h)
         return h
 
+    # -- hybrid stacks with convolved sublayer inputs and a learned average over depth ---------------------------------
+    def _canon_layers(self, batch: StepBatch, h: torch.Tensor, ids: torch.Tensor) -> torch.Tensor:
+        """x <- x + mixer(g), x <- x + ff(g) with g = n + causal_conv(n), n the sublayer's norm of x; what goes on from a layer
+        is the weighted sum of the embedding and of all layers' results. Linear attention (decays per head or per key channel),
+        latent attention (window, latents shared between layers); dense PolyNorm or routed feed-forward (experts by token id,
+        gated shared expert). Norms, convolutions, rotations, scores, decays, states and the residual sum are fp32 whatever
+        the dtype."""
+        from .rope import rope_table
+        spec, dt, eps, w = self.spec, self.dtype, self.spec.norm_eps, self.w
+        T, dev = h.shape[0], self.device
+        F = torch.nn.functional
+        lin = lambda x, m: R.gemm(x.to(dt), m, None, None, 0)
+        rnd = lambda x: x.to(dt).float()
+        seqs, t0 = [], 0
+        for slot, qlen, ctx in zip(batch.slots, batch.q_lens, batch.ctx_lens):
+            if qlen > 0 and ctx == 0:
+                self.cache.pop(slot, None)            # a sequence's first tokens: whatever the slot held before is void
+            if qlen > 0:
+                seqs.append((slot, t0, qlen, ctx))
+            t0 += qlen
+        pos = torch.tensor([c + i for c, q in zip(batch.ctx_lens, batch.q_lens) for i in range(q)], dtype=torch.long, device=dev)
+        far = int(pos.max()) + 1 if T else 1
+
+        def read(x, norm_w, taps, li, which):
+            """What a sublayer reads: the norm of x plus its convolution (`which`: -2 mixer, -1 feed-forward)."""
+            n = R.rmsnorm(x, norm_w, eps, unit_offset=True)
+            if not spec.input_conv:
+                return n
+            g = torch.empty_like(n)
+            for slot, s0, qlen, _ in seqs:
+                st = self._slot_cache(slot)[li]
+                y, st[which] = R.short_conv(n[s0:s0 + qlen], st[which], taps)
+                g[s0:s0 + qlen] = n[s0:s0 + qlen] + y
+            return g
+
+        results = [h]
+        self.layer_outputs = []
+        for li, l in enumerate(w.layers):
+            ls = spec.layer_specs[self.plan.layers[li]]
+            H, d, dv = ls.heads, ls.dim, ls.vdim
+            g = read(h, l["ln1_w"], l.get("conv1"), li, -2)
+            z = lin(g, l["w_in"])
+            mixed = torch.empty(T, H, dv, dtype=torch.float32, device=dev)
+            if ls.kind == "linear_attention":
+                qn, vn = H * d, H * dv
+                q, k, v = z[:, :qn].reshape(T, H, d) * ls.scale, z[:, qn:2 * qn].reshape(T, H, d), z[:, 2 * qn:2 * qn + vn].reshape(T, H, dv)
+                gate = z[:, 2 * qn + vn:2 * qn + 2 * vn]
+                if ls.head_decay:
+                    ld = torch.log(torch.tensor(ls.head_decay, dtype=torch.float64)).float().to(dev).view(1, H, 1).expand(T, H, d)
+                else:
+                    ld = (F.logsigmoid(z[:, 2 * qn + 2 * vn:] @ l["w_a2"].float().t() + l["b_a"].float()) / ls.tau).reshape(T, H, d)
+                for slot, s0, qlen, ctx in seqs:
+                    st, sl = self._slot_cache(slot)[li], slice(s0, s0 + qlen)
+                    mixed[sl], st[0] = R.linear_attention(q[sl], k[sl], v[sl], ld[sl], st[0])
+                mixed = R.rmsnorm(mixed, l["o_norm_w"] if ls.o_norm else torch.ones(dv, device=dev), eps).reshape(T, vn) * F.silu(gate)
+            else:
+                dr, Rk = ls.rot_dim, ls.kv_rank
+                q = z[:, :H * (d + dr)].reshape(T, H, d + dr)
+                own = ls.kv_from < 0
+                if ls.rope_dims:
+                    cos, sin = rope_table(ls.rope_dims, ls.rope_base, ls.rope_scaling, far, dev)
+                    q = torch.cat([q[..., :d], R.rope_partial(q[..., d:], cos, sin, pos, ls.rope_interleaved)], dim=-1)
+                if own:
+                    c, kr = R.rmsnorm(z[:, H * (d + dr):H * (d + dr) + Rk], l["dkv_norm"], eps), z[:, H * (d + dr) + Rk:].reshape(T, 1, dr)
+                    if ls.rope_dims:
+                        kr = R.rope_partial(kr, cos, sin, pos, ls.rope_interleaved)
+                for slot, s0, qlen, ctx in seqs:
+                    st, sl = self._slot_cache(slot)[li if own else ls.kv_from], slice(s0, s0 + qlen)
+                    if own:
+                        assert st[0].shape[0] >= ctx, f"slot {slot}: cache has {st[0].shape[0]} tokens, step says {ctx}"
+                        st[0] = torch.cat([st[0][:ctx], c[sl].reshape(qlen, 1, Rk).to(dt)])
+                        st[1] = torch.cat([st[1][:ctx], kr[sl].to(dt)])
+                    n_all = st[0].shape[0]
+                    ku, vv = lin(st[0][:, 0], l["w_uk"]).reshape(n_all, H, d), lin(st[0][:, 0], l["w_uv"]).reshape(n_all, H, dv)
+                    kk = torch.cat([ku, st[1].float().expand(n_all, H, dr)], dim=-1)
+                    mixed[sl] = R.attention(q[sl], kk, vv, ctx, ls.scale, window=ls.window or 0)
+                mixed = mixed.reshape(T, H * dv)
+            h = h + lin(mixed, l["w_o"])
+            if ls.has_ff:
+                g = read(h, l["ln2_w"], l.get("conv2"), li, -1)
+                if ls.moe is None:
+                    y = lin(rnd(R.poly_norm(lin(g, l["w_up"]), l["act"], eps)), l["w_down"])
+                else:
+                    e = ls.moe
+
+                    def glu(x, g_, u_, d_, limit, scale=None):
+                        a, u = lin(x, g_).clamp(max=limit), lin(x, u_).clamp(min=-limit, max=limit)
+                        act = a * torch.sigmoid(1.702 * a) * (u + 1.0)
+                        return lin(rnd(act if scale is None else act * scale), d_)
+
+                    idx = l["table"].long()[ids]
+                    y = torch.zeros_like(h)
+                    for ex in range(e.experts):
+                        rows = (idx == ex).any(-1).nonzero(as_tuple=True)[0]
+                        if rows.numel():
+                            y.index_add_(0, rows, glu(g[rows], l["w_gate_e"][ex], l["w_up_e"][ex], l["w_down_e"][ex], e.limit) / e.top)
+                    if e.shared_ff:
+                        y = y + glu(g, l["w_gate_s"], l["w_up_s"], l["w_down_s"], e.shared_limit, torch.sigmoid(lin(g, l["w_sg"])) if e.shared_gate else None)
+                h = h + y
+            if spec.depth_average:
+                results.append(h)
+                h = sum(cj * r for cj, r in zip(l["dwa"].float(), results))
+            self.layer_outputs.append(h)
+        return h
+
     def _forward_hybrid(self, batch: StepBatch, x: torch.Tensor) -> torch.Tensor:
         T = batch.num_tokens
         ids = torch.as_tensor(x).to(self.device).long().reshape(-1)
         assert ids.numel() == T, f"expected {T} token ids, got {ids.numel()}"
+        if self.spec.input_conv or self.spec.depth_average:
+            h = self._canon_layers(batch, self.w.embed[ids].float(), ids)
+            self.last_hidden = h
+            rows = self._out_rows(batch)
+            if not rows:
+                return torch.empty(0, self.spec.vocab_size, dtype=torch.float32, device=self.device)
+            hn = R.rmsnorm(h[rows], self.w.final_norm_w, self.spec.norm_eps, unit_offset=True)
+            return R.gemm(hn.to(self.dtype), self.w.lm_head).float()
         if self.spec.post_norm:
             h = self._postnorm_layers(batch, self.w.embed[ids].float())
             self.last_hidden = h

@@ -457,6 +457,157 @@ def _random_zovozen_weights(spec: ModelSpec, plan: StagePlan, seed: int, device,
     return w
 
 
+# ---- Pifutar: checkpoint names <-> the logical layout ---------------------------------------------------------------
+# Per layer: ln1_w, ln2_w norms (stored as the distance from one), conv1, conv2 [H, taps] input convolutions, dwa [layer + 2]
+#   linear attention: w_in = q | k | v | g (| a1), w_o; decays per channel: w_a2 [heads dim, rank], b_a; o_norm_w [vdim]
+#   latent attention: w_in = q (| dkv), w_uk, w_uv, w_o; dkv_norm
+#   dense: w_up, w_down, act [4]      moe: w_gate_e / w_up_e [E, ff, H], w_down_e [E, H, ff], table [vocab, top] (integers),
+#   w_gate_s, w_up_s, w_down_s, w_sg [1, H]
+def _pifutar_layer_names(ls, p: str, taps: int) -> Dict[str, object]:
+    """logical name -> checkpoint name(s); a tuple is concatenated along the rows, a list stacked."""
+    m, f = p + "mix.", p + "mlp."
+    n: Dict[str, object] = {"ln1_w": p + "norm1", "dwa": p + "dwa", "w_o": m + "o"}
+    if taps:
+        n["conv1"] = p + "canon1"
+    if ls.kind == "linear_attention":
+        n["w_in"] = tuple(m + x for x in ("q", "k", "v", "g") + (() if ls.head_decay else ("a1",)))
+        if not ls.head_decay:
+            n["w_a2"], n["b_a"] = m + "a2", m + "a2.b"
+        if ls.o_norm:
+            n["o_norm_w"] = m + "norm"
+    else:
+        n["w_in"] = (m + "q",) if ls.kv_from >= 0 else (m + "q", m + "dkv")
+        n["w_uk"], n["w_uv"] = m + "uk", m + "uv"
+        if ls.kv_from < 0:
+            n["dkv_norm"] = m + "dkv.norm"
+    if ls.has_ff:
+        n["ln2_w"] = p + "norm2"
+        if taps:
+            n["conv2"] = p + "canon2"
+    if ls.moe is not None:
+        for x in ("gate", "up", "down"):
+            n[f"w_{x}_e"] = [f"{f}e{j}.{x}" for j in range(ls.moe.experts)]
+            if ls.moe.shared_ff:
+                n[f"w_{x}_s"] = f"{f}shared.{x}"
+        n["table"] = f + "table"
+        if ls.moe.shared_gate:
+            n["w_sg"] = f + "shared.sg"
+    elif ls.ff:
+        n["w_up"], n["w_down"], n["act"] = f + "up", f + "down", f + "act"
+    return n
+
+
+def _pifutar_in_sizes(ls, rank: int) -> List[int]:
+    """Rows of the parts of w_in; `rank` is the rank of the decay projection (a checkpoint's tensors say it)."""
+    if ls.kind == "linear_attention":
+        return [ls.heads * ls.dim, ls.heads * ls.dim, ls.heads * ls.vdim, ls.heads * ls.vdim] + ([] if ls.head_decay else [rank])
+    return [ls.heads * (ls.dim + ls.rot_dim)] + ([ls.kv_rank + ls.rot_dim] if ls.kv_from < 0 else [])
+
+
+def _load_pifutar_weights(rd, spec: ModelSpec, plan: StagePlan, device, dtype) -> StageWeights:
+    w = StageWeights(spec, plan)
+    H = spec.hidden_size
+
+    def get(name):
+        t = rd.get(name)
+        return t.to(device=device, dtype=dtype if t.is_floating_point() else torch.int32)
+
+    w.embed, w.final_norm_w = get("embed"), get("final.norm")
+    w.lm_head = w.embed
+    for i in plan.layers:
+        ls, l = spec.layer_specs[i], {}
+        for k, names in _pifutar_layer_names(ls, f"l{i}.", spec.input_conv).items():
+            if isinstance(names, tuple):
+                l[k] = torch.cat([get(x) for x in names], dim=0)
+            elif isinstance(names, list):
+                l[k] = torch.stack([get(x) for x in names], dim=0)
+            else:
+                l[k] = get(names)
+        rank = int(l["w_a2"].shape[1]) if "w_a2" in l else 0
+        want = {"w_in": (sum(_pifutar_in_sizes(ls, rank)), H), "w_o": (H, ls.heads * ls.vdim), "dwa": (i + 2,), "ln1_w": (H,),
+                "conv1": (H, spec.input_conv), "conv2": (H, spec.input_conv), "w_a2": (ls.heads * ls.dim, rank), "b_a": (ls.heads * ls.dim,),
+                "o_norm_w": (ls.vdim,), "w_uk": (ls.heads * ls.dim, ls.kv_rank), "w_uv": (ls.heads * ls.vdim, ls.kv_rank),
+                "w_up": (ls.ff, H), "w_down": (H, ls.ff), "act": (4,)}
+        if ls.moe is not None:
+            e = ls.moe
+            want.update({"w_gate_e": (e.experts, e.ff, H), "w_down_e": (e.experts, H, e.ff), "table": (spec.vocab_size, e.top),
+                         "w_gate_s": (e.shared_ff, H), "w_sg": (1, H)})
+            if int(l["table"].min()) < 0 or int(l["table"].max()) >= e.experts:
+                raise ValueError(f"layer {i}: the expert table names experts beyond {e.experts}")
+        for k, shape in want.items():
+            if k in l and tuple(l[k].shape) != shape:
+                raise ValueError(f"layer {i}: {k} has the shape {tuple(l[k].shape)}, the config says {shape}")
+        w.layers.append(l)
+    return w
+
+
+def export_pifutar_state_dict(w: StageWeights) -> Dict[str, torch.Tensor]:
+    """Logical -> checkpoint names (tests, `save` of random models)."""
+    spec = w.spec
+    sd = {"embed": w.embed, "final.norm": w.final_norm_w}
+    for i, l in zip(w.plan.layers, w.layers):
+        ls = spec.layer_specs[i]
+        rank = int(l["w_a2"].shape[1]) if "w_a2" in l else 0
+        for k, names in _pifutar_layer_names(ls, f"l{i}.", spec.input_conv).items():
+            if isinstance(names, tuple):
+                for x, t in zip(names, torch.split(l[k], _pifutar_in_sizes(ls, rank))):
+                    sd[x] = t
+            elif isinstance(names, list):
+                for x, t in zip(names, l[k]):
+                    sd[x] = t
+            else:
+                sd[names] = l[k]
+    return {k: v.detach().clone().contiguous() for k, v in sd.items()}
+
+
+def _random_pifutar_weights(spec: ModelSpec, plan: StagePlan, seed: int, device, dtype) -> StageWeights:
+    """Random weights with which every mechanism matters: projections at 1 / sqrt(fan-in), convolution taps, depth weights and
+    polynomial coefficients of order one, decays that span short and long memories."""
+    H, V = spec.hidden_size, spec.vocab_size
+    w = StageWeights(spec, plan)
+    rn = lambda name, shape, std: _randn(name, shape, seed, device, dtype, std=std)
+    w.embed, w.final_norm_w = rn("embed", (V, H), 1.0), rn("final.norm", (H,), 0.1)
+    w.lm_head = w.embed
+    for i in plan.layers:
+        ls, p = spec.layer_specs[i], f"layers.{i}."
+        on, R = ls.heads * ls.vdim, ls.kv_rank
+        rank = 0 if ls.kind != "linear_attention" or ls.head_decay else (ls.rank or 16)
+        l: Dict[str, torch.Tensor] = {"ln1_w": rn(p + "ln1_w", (H,), 0.1), "w_in": rn(p + "w_in", (sum(_pifutar_in_sizes(ls, rank)), H), H ** -0.5),
+                                      "w_o": rn(p + "w_o", (H, on), on ** -0.5)}
+        # (the weights of a depth average sum to about one, most of it on the latest result)
+        l["dwa"] = rn(p + "dwa", (i + 2,), 0.3 / (i + 2)) + torch.tensor([0.3 / (i + 1)] * (i + 1) + [0.7], device=device, dtype=dtype)
+        if spec.input_conv:
+            l["conv1"] = rn(p + "conv1", (H, spec.input_conv), 0.3)
+        if rank:
+            l["w_a2"], l["b_a"] = rn(p + "w_a2", (ls.heads * ls.dim, rank), rank ** -0.5), rn(p + "b_a", (ls.heads * ls.dim,), 1.0)
+        if ls.o_norm:
+            l["o_norm_w"] = torch.ones(ls.vdim, device=device, dtype=dtype) + rn(p + "o_norm_w", (ls.vdim,), 0.1)
+        if ls.kind == "latent_attention":
+            l["w_uk"], l["w_uv"] = rn(p + "w_uk", (ls.heads * ls.dim, R), R ** -0.5), rn(p + "w_uv", (on, R), R ** -0.5)
+            if ls.kv_from < 0:
+                l["dkv_norm"] = torch.ones(R, device=device, dtype=dtype) + rn(p + "dkv_norm", (R,), 0.1)
+        if ls.has_ff:
+            l["ln2_w"] = rn(p + "ln2_w", (H,), 0.1)
+            if spec.input_conv:
+                l["conv2"] = rn(p + "conv2", (H, spec.input_conv), 0.3)
+        if ls.moe is not None:
+            e = ls.moe
+            l["w_gate_e"], l["w_up_e"] = rn(p + "w_gate_e", (e.experts, e.ff, H), 1.5 * H ** -0.5), rn(p + "w_up_e", (e.experts, e.ff, H), 1.5 * H ** -0.5)
+            l["w_down_e"] = rn(p + "w_down_e", (e.experts, H, e.ff), e.ff ** -0.5)
+            g = torch.Generator().manual_seed(_seed_for(p + "table", seed))
+            l["table"] = torch.argsort(torch.rand(V, e.experts, generator=g), dim=-1)[:, :e.top].to(device=device, dtype=torch.int32).contiguous()
+            if e.shared_ff:
+                l["w_gate_s"], l["w_up_s"] = rn(p + "w_gate_s", (e.shared_ff, H), H ** -0.5), rn(p + "w_up_s", (e.shared_ff, H), H ** -0.5)
+                l["w_down_s"] = rn(p + "w_down_s", (H, e.shared_ff), e.shared_ff ** -0.5)
+            if e.shared_gate:
+                l["w_sg"] = rn(p + "w_sg", (1, H), H ** -0.5)
+        elif ls.ff:
+            l["w_up"], l["w_down"] = rn(p + "w_up", (ls.ff, H), H ** -0.5), rn(p + "w_down", (H, ls.ff), ls.ff ** -0.5)
+            l["act"] = torch.tensor([0.6, 0.4, 0.5, 0.1], device=device, dtype=dtype) + rn(p + "act", (4,), 0.2)
+        w.layers.append(l)
+    return w
+
+
 def _random_hybrid_weights(spec: ModelSpec, plan: StagePlan, seed: int, device, dtype) -> StageWeights:
     """Random weights of a hybrid stack, scaled so that activations stay of order one through any depth
     (projections at 1 / sqrt(fan-in), embedding at one) and every bias, convolution tap and gate matters."""
@@ -466,6 +617,8 @@ def _random_hybrid_weights(spec: ModelSpec, plan: StagePlan, seed: int, device, 
         return _random_tezesun_weights(spec, plan, seed, device, dtype)
     if spec.family == "zovozen":
         return _random_zovozen_weights(spec, plan, seed, device, dtype)
+    if spec.family == "pifutar":
+        return _random_pifutar_weights(spec, plan, seed, device, dtype)
     H, V = spec.hidden_size, spec.vocab_size
     w = StageWeights(spec, plan)
     rn = lambda name, shape, std: _randn(name, shape, seed, device, dtype, std=std)
@@ -505,6 +658,8 @@ def _load_hybrid_weights(rd, spec: ModelSpec, plan: StagePlan, device, dtype) ->
         return _load_tezesun_weights(rd, spec, plan, device, dtype)
     if spec.family == "zovozen":
         return _load_zovozen_weights(rd, spec, plan, device, dtype)
+    if spec.family == "pifutar":
+        return _load_pifutar_weights(rd, spec, plan, device, dtype)
     w = StageWeights(spec, plan)
     get = lambda name: rd.get(name).to(device=device, dtype=dtype)
     if plan.has_embed or plan.has_head:

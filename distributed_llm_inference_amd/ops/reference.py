@@ -194,6 +194,24 @@ def moe_route(scores: torch.Tensor, top: int, groups: int, keep: int, scale: flo
     return idx, val / (val.sum(-1, keepdim=True) + 1e-20) * scale
 
 
+def linear_attention(q, k, v, log_decay, S):
+    """Token by token, per head: S <- diag(exp(log_decay)) S + k v^T; o = S^T q. q, k, log_decay [T, H, d], v [T, H, dv],
+    S [H, d, dv] fp32. Returns (o [T, H, dv], S)."""
+    qf, kf, vf, a, S = q.float(), k.float(), v.float(), torch.exp(log_decay.float()), S.float().clone()
+    out = torch.empty_like(vf)
+    for t in range(qf.shape[0]):
+        S = a[t].unsqueeze(2) * S + kf[t].unsqueeze(2) * vf[t].unsqueeze(1)
+        out[t] = torch.einsum("hdv,hd->hv", S, qf[t])
+    return out, S
+
+
+def poly_norm(z: torch.Tensor, coef: torch.Tensor, eps: float) -> torch.Tensor:
+    """a N(z) + b N(z^2) + c N(z^3) + e for coef = (a, b, c, e); N divides a row by its root mean square."""
+    zf, c = z.float(), coef.float()
+    unit = lambda x: x * torch.rsqrt(x.pow(2).mean(-1, keepdim=True) + eps)
+    return c[0] * unit(zf) + c[1] * unit(zf * zf) + c[2] * unit(zf * zf * zf) + c[3]
+
+
 def xielu(z: torch.Tensor, p, q) -> torch.Tensor:
     """z > 0: softplus(p) z^2 + z / 2; z <= 0: (1/2 + softplus(q)) (exp(z) - 1 - z) + z / 2."""
     zf = z.float()
