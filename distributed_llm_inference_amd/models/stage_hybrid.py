@@ -54,6 +54,20 @@ Stacks that norm their sublayers' OUTPUTS only (`spec.post_norm`: the sublayers 
                   the identity experts' share of x;  silu(gate) * up -> shared down GEMM ]
              -> x += rms(ff) w
 
+Stacks with convolved sublayer inputs and a learned average over depth (`spec.input_conv`, `spec.depth_average`) run through
+`_layers_canon`: per layer
+
+    x (fp32) -> rms factor, g = h + causal conv(h) (single-token steps: in the join below; else one more kernel)
+             -> ONE input GEMM (all projections of the mixer)
+             -> [ linear attention with decays per head or per key channel: state update / chunked scan, head norm and gate
+                | latent norm + rotation + cache write (layers that read another layer's rows: rotation of q alone)
+                  -> key up-projection absorbed into the query -> attention over the latent rows (window) -> value up-projection ]
+             -> o GEMM -> join (x += y, the next rms factor and input; the closing sublayer's last h saved in the slot's ring)
+             -> [ up GEMM -> PolyNorm -> down GEMM
+                | the experts' GEMMs over the rows the plan sorted by token id (all routed layers' plans: one launch ahead of the
+                  layers);  shared gate | up | sigmoid gate GEMM -> activation -> shared down GEMM ]
+             -> join (x += experts + shared, kept as X_(i+1), x <- sum_j c_j X_j, the next layer's factor and input)
+
 Matrix products take bf16 operands (or fp32: `dtype="fp32"`, everything in true 32-bit) and accumulate in
 fp32; norms, scores, softmax, value mixing, gates, decays and states are fp32 in both modes.
 """
@@ -154,7 +168,15 @@ class HybridGpuStage(GpuStage):
         self.gated = spec.norm_kind == "dyt"
         self.par = spec.parallel_block
         self.post = spec.post_norm
+        self.canon = spec.input_conv > 0 or spec.depth_average
         self.runs = spec.layer_runs()
+        if self.canon:
+            self.mfma_attn = [False] * len(self.specs)
+            # attention over the latent rows on the matrix cores in bf16 where the row and the latent come in whole 16-byte pieces;
+            # other sizes, and the fp32 mode, on the one-wave-per-(token, head) kernel. DLIA_CANON_TILE_ATTN=0: all on that (A/B)
+            tile_ok = dtype == "bf16" and os.environ.get("DLIA_CANON_TILE_ATTN", "1") != "0"
+            self._tile = [tile_ok and ls.kind == "latent_attention" and self._score_dim(ls) % 8 == 0 for ls in self.specs]
+            self._load_canon(weights, f32, mat)
         if self.post:
             self.mfma_attn = [False] * len(self.specs)
             self._attn_of_run = [ls.branches[0] for ls in self.specs]
@@ -173,7 +195,7 @@ class HybridGpuStage(GpuStage):
                             bool(self.K.mixed_attention_fits(a.heads, a.kv_heads, a.dim, a.vdim))
                             for a, tile in zip(self._attn_of_run, self._tile)]
             self._load_post(weights, f32, mat)
-        if self.post:
+        if self.post or self.canon:
             pass
         elif self.par:
             self.mfma_attn = [False] * len(self.specs)
@@ -244,6 +266,11 @@ class HybridGpuStage(GpuStage):
             if ls.kind == "rglru":
                 st += (torch.zeros(max_slots + 1, max(ls.conv - 1, 1), ls.rec_width, device=dev), torch.zeros(max_slots + 1, ls.rec_width, device=dev))
             self.rec.append(st)
+        for ls in (self.specs if self.canon else []):
+            # rings of the last taps - 1 inputs of both sublayers' convolutions, and a linear attention's state
+            ring = lambda: torch.zeros(max_slots + 1, spec.input_conv - 1, spec.hidden_size, device=dev) if spec.input_conv > 1 else None
+            st = torch.zeros(max_slots + 1, ls.heads, ls.dim, ls.vdim, device=dev) if ls.kind == "linear_attention" else None
+            self.rec.append((ring(), ring() if ls.has_ff else None, st))
         for ls in (self.specs if self.post else []):
             # the matrix memory's state (its normaliser as one more column) and running maxima
             b = ls.branches[1]
@@ -256,7 +283,7 @@ class HybridGpuStage(GpuStage):
                 b = ls.branches[1]
                 self.rec.append((torch.zeros(max_slots + 1, b.heads, b.dim, b.vdim + 1, device=dev),
                                  torch.zeros(max_slots + 1, b.heads, 128, device=dev)))
-        for ls in ([] if (self.gated or self.par or self.post) else self.specs):
+        for ls in ([] if (self.gated or self.par or self.post or self.canon) else self.specs):
             if ls.kind == "delta":
                 C = 2 * ls.kv_heads * ls.dim + ls.heads * ls.vdim
                 self.rec.append((torch.zeros(max_slots + 1, max(ls.conv - 1, 1), C, device=dev),
@@ -311,6 +338,8 @@ class HybridGpuStage(GpuStage):
 
     # ---- workspaces ---------------------------------------------------------------------------------------
     def _new_work(self, rows: int):
+        if self.canon:
+            return self._new_work_canon(rows)
         if self.post:
             return self._new_work_post(rows)
         if self.par:
@@ -346,13 +375,13 @@ class HybridGpuStage(GpuStage):
     # ---- cache and state sizing -------------------------------------------------------------------------
     def kv_block_bytes(self) -> int:
         e = 4 if self.act_dtype == torch.float32 else 2
-        if self.par:
-            return max(1, sum(BLOCK * e * sum(self._par_rows(li)) for li, ls in enumerate(self.specs) if ls.kind != "rglru"))
+        if self.par or self.canon:
+            return max(1, sum(BLOCK * e * sum(self._par_rows(li)) for li, ls in enumerate(self.specs) if self._keeps_rows(ls)))
         return max(1, sum(ls.kv_heads * BLOCK * (ls.dim + ls.vdim) * e for ls in self._attn_of_run if ls is not None))
 
     def _decode_state_bytes(self) -> int:
         n = 0
-        if self.gated or self.par or self.post:
+        if self.gated or self.par or self.post or self.canon:
             per_row = sum(t.numel() * t.element_size() for t in vars(self.wk0).values() if torch.is_tensor(t)) // self.max_tokens
             return sum(B * (per_row + 4 * self.vocab_pad) for B in self.graph_sizes)
         for B in self.graph_sizes:
@@ -375,12 +404,12 @@ class HybridGpuStage(GpuStage):
                     torch.zeros(self.num_blocks, G, BLOCK, a.vdim, device=dev, dtype=at)
                 self.kv.append((kc, vc))
             return
-        if self.par:
+        if self.par or self.canon:
             # attention: key rows hold a head's score maps side by side, value rows apart; latent attention: ONE row per token,
             # the normed latent followed by the rotated key part (the values are the row's first entries)
             self.kv = []
             for li, ls in enumerate(self.specs):
-                if ls.kind == "rglru":
+                if not self._keeps_rows(ls):      # (a recurrent layer, or one that reads another layer's rows)
                     self.kv.append(None)
                     continue
                 kr, vr = self._par_rows(li)
@@ -417,6 +446,12 @@ class HybridGpuStage(GpuStage):
 
     # ---- the layer stack ----------------------------------------------------------------------------------
     def _embed_rows(self, wk, T: int, ids, pos):
+        if self.canon:
+            self.K.embed32(wk.hist[0][:T], ids, self.embed)
+            if self._plan_rows:
+                self.K.moe_table_plan(wk.tiles, wk.row_tok, wk.pair_row, self.tables, ids, wk.plan_dev, wk.plan_host, T, self.spec.vocab_size,
+                                      self.BIG_PAIRS)
+            return
         if self.pos_embed is not None:
             self.K.embed_pos32(wk.h[:T], ids, pos, self.embed, self.pos_embed)
         else:
@@ -424,6 +459,8 @@ class HybridGpuStage(GpuStage):
 
     def _layers(self, wk: _HybridWork, T: int, B: int, tok_pos, tok_seq, q_start, ctx, slots, max_q: int, splits: int,
                 alone: bool = False, lead_decode: int = 0):
+        if self.canon:
+            return self._layers_canon(wk, T, B, tok_pos, tok_seq, q_start, ctx, slots, max_q)
         if self.post:
             return self._layers_post(wk, T, B, tok_pos, tok_seq, q_start, ctx, slots, max_q)
         if self.par:
@@ -707,6 +744,11 @@ class HybridGpuStage(GpuStage):
     def _score_dim(ls) -> int:
         """Entries of one score map's keys."""
         return ls.kv_rank + ls.rot_dim if ls.kind == "latent_attention" else ls.dim
+
+    @staticmethod
+    def _keeps_rows(ls) -> bool:
+        """The layer has a paged cache of its own."""
+        return ls.kind in ("attention", "latent_attention") and ls.kv_from < 0
 
     def _par_rows(self, li: int) -> tuple:
         """(entries of a token's key row, of its value row) in the cache of attention layer li, over all its key / value heads.
@@ -1080,6 +1122,222 @@ class HybridGpuStage(GpuStage):
                 self.layer_outputs.append(h.clone())
         return None
 
+    # ---- stacks with convolved sublayer inputs and a learned average over depth ----------------------------------------
+    BIG_PAIRS = 1024             # routed pairs of a step from which the experts run on 128-row tiles
+
+    def _load_canon(self, weights: StageWeights, f32, mat):
+        """Device weights of the stack. A mixer's input projections are ONE matrix, the shared expert's gate | up | sigmoid gate
+        another. What norms, convolutions, depth averages, decays and the polynomial need stays fp32 in both modes; the decay
+        projection's second factor is kept in fp32, transposed, for the recurrence's own kernels."""
+        from .rope import rope_table
+        spec, dev = self.spec, self.device
+        H = spec.hidden_size
+        if H > int(self.K.stream_join_max_width(H % 4 == 0)):
+            raise ValueError(f"width {H} is beyond what the row kernels take")
+        self.embed, self.pos_embed = mat(weights.embed), None
+        self.lm_head, self.lm_head_p = self.embed, None
+        self.final_norm_w = f32(weights.final_norm_w)
+        self.vocab_pad = packing.padded_n(spec.vocab_size)
+        self.layers = []
+        ropes: Dict[tuple, tuple] = {}
+        tables = []
+        self._plan_rows = []                 # per routed layer: (table offset, chosen, experts, 128-row tiles allowed)
+        for i, ls in enumerate(self.specs):
+            l = weights.layers[i]
+            p: Dict[str, object] = {"ln1_w": f32(l["ln1_w"]), "dwa": f32(l["dwa"]) if spec.depth_average else None, "plan": -1}
+            p["conv1"] = f32(l["conv1"].t()) if spec.input_conv else None          # [taps, width]
+            self._matrix(p, "w_in", mat(l["w_in"]), None)
+            self._matrix(p, "w_o", mat(l["w_o"]), None)
+            if ls.kind == "linear_attention":
+                p["decay"] = p["a2t"] = p["b_a"] = None
+                if ls.head_decay:
+                    # the decays as they are for single tokens, their logarithms (formed in float64) for chunks
+                    dd = torch.tensor(ls.head_decay, dtype=torch.float64)
+                    p["decay"] = torch.stack([dd, torch.log2(dd)]).float().to(dev).contiguous()
+                else:
+                    p["a2t"], p["b_a"] = f32(l["w_a2"].t()), f32(l["b_a"])
+                p["o_norm_w"] = f32(l["o_norm_w"]) if ls.o_norm else None
+            else:
+                Hh, d, dr, dv, R = ls.heads, ls.dim, ls.rot_dim, ls.vdim, ls.kv_rank
+                p["dkv_norm"] = f32(l["dkv_norm"]) if ls.kv_from < 0 else None
+                # q . (W_uk c) = (W_uk^T q) . c: the key up-projection moves to the query's side, the cache keeps the latent alone
+                wa = torch.zeros(Hh, R + dr, d + dr, device=dev, dtype=self.act_dtype)
+                wa[:, :R, :d] = mat(l["w_uk"]).reshape(Hh, d, R).transpose(1, 2)
+                wa[:, R:, d:] = torch.eye(dr, device=dev, dtype=self.act_dtype)
+                p["w_abs"], p["w_uv"] = wa.contiguous(), mat(l["w_uv"]).reshape(Hh, dv, R).contiguous()
+                p["cos"] = p["sin"] = None
+                if ls.rope_dims:
+                    key = (ls.rope_dims, ls.rope_base, ls.rope_scaling)
+                    if key not in ropes:
+                        ropes[key] = tuple(t.contiguous() for t in rope_table(ls.rope_dims, ls.rope_base, ls.rope_scaling, self.max_seq_len, dev))
+                    p["cos"], p["sin"] = ropes[key]
+            if ls.has_ff:
+                p["ln2_w"], p["conv2"] = f32(l["ln2_w"]), f32(l["conv2"].t()) if spec.input_conv else None
+            if ls.moe is not None:
+                e = ls.moe
+                if e.experts > 1024:
+                    raise ValueError(f"layer {i}: up to 1024 experts are supported")
+                p["plan"] = len(self._plan_rows)
+                big = self.wmode == "bf16" and H % 32 == 0 and e.ff % 32 == 0
+                self._plan_rows.append((sum(t.numel() for t in tables), e.top, e.experts, big))
+                tables.append(l["table"].to(device=dev, dtype=torch.int32).contiguous().reshape(-1))
+                p["w_gate_e"], p["w_up_e"], p["w_down_e"] = (mat(l[k]) for k in ("w_gate_e", "w_up_e", "w_down_e"))
+                if e.shared_ff:
+                    self._matrix(p, "w_ff", torch.cat([mat(l["w_gate_s"]), mat(l["w_up_s"])] + ([mat(l["w_sg"])] if e.shared_gate else [])), None)
+                    self._matrix(p, "w_down_s", mat(l["w_down_s"]), None)
+            elif ls.ff:
+                self._matrix(p, "w_up", mat(l["w_up"]), None)
+                self._matrix(p, "w_down", mat(l["w_down"]), None)
+                p["act"] = f32(l["act"])
+            self.layers.append(p)
+            weights.layers[i] = {}
+        self.tables = torch.cat(tables) if tables else None
+        if self._packed and H % 128 == 0:
+            self.lm_head_p = packing.pack_weight(self.lm_head)
+            self._shapes.append((self.vocab_pad, H, False))
+
+    def _moe_tiles(self, rows: int, pl: tuple) -> tuple:
+        """(rows per tile, tiles at most) of a routed layer in a step of `rows` tokens."""
+        _, top, experts, big = pl
+        tr = 128 if big and rows * top >= self.BIG_PAIRS else 32
+        return tr, (rows * top + tr - 1) // tr + experts
+
+    def _new_work_canon(self, rows: int):
+        s, dev, at = self.spec, self.device, self.act_dtype
+        z = lambda n, dt=torch.float32: torch.zeros(max(int(n), 1), device=dev, dtype=dt)
+        B, H = min(rows, self.max_batch), s.hidden_size
+        portions = not hasattr(self, "wk0")          # (the fixed-shape decode states run single-token steps only)
+        zc = mc = yc = sc = z2 = ac = q16 = qa = ol = part = lin = ef = erows = 1
+        for ls, p, tile in zip(self.specs, self.layers, self._tile):
+            zc, yc, mc = max(zc, self._cols(p, "w_in")), max(yc, self._cols(p, "w_o")), max(mc, ls.heads * ls.vdim)
+            if ls.kind == "linear_attention":
+                if portions:
+                    lin = max(lin, int(self.K.linear_attention_ws_floats(rows, B, ls.heads, ls.dim, ls.vdim, not ls.head_decay)))
+            else:
+                q16, qa, ol = max(q16, ls.heads * (ls.dim + ls.rot_dim)), max(qa, ls.heads * (ls.kv_rank + ls.rot_dim)), max(ol, ls.heads * ls.kv_rank)
+                if tile:          # (key splits of single-token steps, of any number of rows up to B)
+                    part = max([part] + [int(self.K.tile_attention_part_floats(b_, ls.heads, 1, ls.kv_rank, 1)) for b_ in range(1, B + 1)])
+            if ls.moe is not None:
+                e = ls.moe
+                for t in {rows, min(rows, (self.BIG_PAIRS - 1) // e.top)}:      # (the most rows of either tile size)
+                    tr, nt = self._moe_tiles(t, self._plan_rows[p["plan"]])
+                    erows, ef = max(erows, tr * nt), max(ef, e.ff)
+                if e.shared_ff:
+                    z2, sc, yc = max(z2, self._cols(p, "w_ff")), max(sc, e.shared_ff), max(yc, self._cols(p, "w_down_s"))
+            elif ls.ff:
+                z2, ac, yc = max(z2, self._cols(p, "w_up")), max(ac, ls.ff), max(yc, self._cols(p, "w_down"))
+        ws_floats = self._ws_floats
+        if self._packed and rows > self.decode_rows:
+            for m_ in {rows, min(rows, 512), min(rows, 1024)}:
+                if m_ > self.decode_rows:
+                    ws_floats = max([ws_floats] + [int(self.K.gemm_ws_floats(m_, n_, k_)) for n_, k_, _ in self._shapes])
+        # where each routed layer's plan lies in the shared lists (room for either tile size)
+        i32, desc, at_t, at_r, at_p = torch.int32, [], 0, 0, 0
+        for pl in self._plan_rows:
+            off, top, experts, big = pl
+            desc.append([off, top, experts, at_t, at_r, at_p, 1 if big else 0, 0])
+            at_t += 1 + (rows * top + 31) // 32 + experts
+            at_r += max(tr * nt for tr, nt in (self._moe_tiles(t, pl) for t in {rows, min(rows, (self.BIG_PAIRS - 1) // top)}))
+            at_p += rows * top
+        host = torch.tensor(desc, dtype=i32).reshape(-1, 8)
+        return SimpleNamespace(
+            h=torch.zeros(rows, H, device=dev), hist=torch.zeros(len(self.specs) + 1 if s.depth_average else 1, rows, H, device=dev), rs=z(rows),
+            xs=torch.zeros(rows, H, device=dev, dtype=at), z=z(rows * zc), mixed=z(rows * mc, at), lin=z(lin),
+            ya=z(rows * yc), yb=z(rows * yc), z2=z(rows * z2), act=z(rows * ac, at), acts=z(rows * sc, at),
+            q16=z(rows * q16, at), qa=z(rows * qa, torch.float32) if not all(t or ls.kind != "latent_attention" for t, ls in zip(self._tile, self.specs)) else z(1),
+            qa16=z(rows * qa if any(self._tile) else 1, at), olat=z(rows * ol, at), part=z(part),
+            tiles=z(at_t, i32), row_tok=z(at_r, i32), pair_row=z(at_p, i32), plan_host=host, plan_dev=host.to(dev), eact=z(erows * ef, at),
+            ey=z(erows * H), ws=z(ws_floats + 4096),
+            head_x=torch.zeros(B, H, device=dev, dtype=at), logits=torch.zeros(B, self.vocab_pad, device=dev), cmax=None, guided=False)
+
+    def _layers_canon(self, wk, T: int, B: int, tok_pos, tok_seq, q_start, ctx, slots, max_q: int):
+        K, spec, eps, H = self.K, self.spec, self.spec.norm_eps, self.spec.hidden_size
+        h, xs, rs, hist = wk.h[:T], wk.xs[:T], wk.rs, wk.hist
+        view = lambda buf, cols: buf[:T * cols].view(T, cols)
+        keep = self.keep_layer_outputs and not torch.cuda.is_current_stream_capturing()
+        if keep:
+            self.layer_outputs = []
+        table, n_layers = self.block_table, len(self.layers)
+        single = max_q == 1
+        closing = [None, None]               # (norm weight, ring) of the sublayer whose output joins next
+
+        def join(x_in, nxt, ya=None, yb=None, ey=None, pairs=None, top=1, result=0, coef=None):
+            """One sublayer boundary. `nxt`: (norm weight, taps, ring) of the sublayer that follows, or None at the end; `result`
+            > 0: the joined stream is X_result, and the average over depth goes on."""
+            nw, taps, ring = nxt or (None, None, None)
+            cw, cring = (None, None) if single else closing
+            K.stream_join(xs if single and nxt else None, h, x_in, ya, yb, ey, pairs, top, 1.0 / top, hist if result else None, result, coef, nw, rs,
+                          cw if cring is not None else None, cring, taps if single and nxt else None, ring if single and nxt else None,
+                          tok_pos, tok_seq, eps)
+            closing[0], closing[1] = nw, ring
+            if nxt and not single:
+                K.canon_conv(xs, h, rs, nw, taps, ring, tok_pos, tok_seq)
+
+        def opening(li):
+            return (self.layers[li]["ln1_w"], self.layers[li]["conv1"], self.rec[li][0]) if li < n_layers else None
+
+        join(hist[0][:T], opening(0))
+        for li, (ls, p) in enumerate(zip(self.specs, self.layers)):
+            Hh, d, dv = ls.heads, ls.dim, ls.vdim
+            z, mixed = view(wk.z, self._cols(p, "w_in")), view(wk.mixed, Hh * dv)
+            self._mm(wk, z, xs, p, "w_in")
+            if ls.kind == "linear_attention":
+                qn, vn = Hh * d, Hh * dv
+                K.linear_attention(mixed, z, self.rec[li][2], p["decay"], p["a2t"], p["b_a"], p["o_norm_w"], q_start, ctx, slots, Hh, d, dv,
+                                   0, qn, 2 * qn, 2 * qn + vn, 2 * qn + 2 * vn, ls.scale, 1.0 / ls.tau, eps, max_q, wk.lin)
+            else:
+                dr, R, tile = ls.rot_dim, ls.kv_rank, self._tile[li]
+                Hq = Hh * (d + dr)
+                kc, vc = self.kv[li if ls.kv_from < 0 else ls.kv_from]
+                q16, olat = view(wk.q16, Hq), view(wk.olat, Hh * R)
+                if ls.kv_from < 0:
+                    K.rope_cache_write(z, Hh, d + dr, d, q16, Hq, z[:, Hq:], R + dr, 1, R + dr, R, 0, R if tile else 0, tile, kc,
+                                       vc if tile else None, ls.rope_dims, ls.rope_interleaved, p["cos"], p["sin"], tok_pos, tok_seq, table,
+                                       p["dkv_norm"], eps)
+                else:
+                    K.rope_rows(z, Hh, d + dr, d, q16, ls.rope_dims, ls.rope_interleaved, p["cos"], p["sin"], tok_pos)
+                if tile:
+                    qa16 = view(wk.qa16, Hh * (R + dr))
+                    K.gemm_blocks(qa16, q16, p["w_abs"], None, d + dr, R + dr)
+                    K.tile_attention(olat, qa16, R + dr, kc, vc, q_start, ctx, slots, table, max_q, Hh, R + dr, R, 1, ls.scale, ls.window or 0, 0,
+                                     0.0, 0.0, 1.0, eps, None, wk.part)
+                else:
+                    qa = view(wk.qa, Hh * (R + dr))
+                    K.gemm_blocks(qa, q16, p["w_abs"], None, d + dr, R + dr)
+                    K.multi_attention(olat, qa, R + dr, kc, kc, 0, tok_pos, tok_seq, table, Hh, R + dr, R, 1, ls.scale, ls.window or 0, 0, 0.0, 0.0,
+                                      1.0, eps, None)
+                K.gemm_blocks(mixed, olat, p["w_uv"], None, R, dv)
+            ya = view(wk.ya, self._cols(p, "w_o"))
+            self._mm(wk, ya, mixed, p, "w_o")
+            ya, yb, ey, pairs, top = ya[:, :H], None, None, None, 1
+            if ls.has_ff:
+                join(h, (p["ln2_w"], p["conv2"], self.rec[li][1]), ya)
+                ya = None
+            if ls.moe is not None:
+                e, pl = ls.moe, wk.plan_host[p["plan"]].tolist()
+                tr, nt = self._moe_tiles(T, self._plan_rows[p["plan"]])
+                tiles, rows, top = wk.tiles[pl[3]:], wk.row_tok[pl[4]:], e.top
+                pairs = wk.pair_row[pl[5]:]
+                eact, ey = wk.eact[:tr * nt * e.ff].view(tr * nt, e.ff), wk.ey[:tr * nt * H].view(tr * nt, H)
+                K.moe_up(eact, xs, p["w_gate_e"], p["w_up_e"], tiles, rows, nt, e.limit, tr)
+                K.moe_down(ey, eact, p["w_down_e"], tiles, rows, nt, tr)
+                if e.shared_ff:
+                    z2, acts, yb = view(wk.z2, self._cols(p, "w_ff")), view(wk.acts, e.shared_ff), view(wk.yb, self._cols(p, "w_down_s"))
+                    self._mm(wk, z2, xs, p, "w_ff")
+                    K.glu_act(acts, z2, e.shared_limit, e.shared_gate)
+                    self._mm(wk, yb, acts, p, "w_down_s")
+                    yb = yb[:, :H]
+            elif ls.ff:
+                z2, act, ya = view(wk.z2, self._cols(p, "w_up")), view(wk.act, ls.ff), view(wk.ya, self._cols(p, "w_down"))
+                self._mm(wk, z2, xs, p, "w_up")
+                K.poly_norm(act, z2, p["act"], eps)
+                self._mm(wk, ya, act, p, "w_down")
+                ya = ya[:, :H]
+            join(h, opening(li + 1), ya, yb, ey, pairs, top, li + 1 if spec.depth_average else 0, p["dwa"])
+            if keep:
+                self.layer_outputs.append(h.clone())
+        return None
+
     def _fold(self, wk, T: int, pend):
         return None
 
@@ -1108,6 +1366,6 @@ class HybridGpuStage(GpuStage):
         size = lambda t: t.numel() * t.element_size()
         wbytes = size(self.embed) + sum(size(t) for l in self.layers for t in l.values() if torch.is_tensor(t))
         kvb = sum(sum(size(t) for t in (kv if isinstance(kv, tuple) else (kv,))) for kv in (self.kv or []) if kv is not None)
-        rec = sum(size(t) for r in self.rec if r is not None for t in r)
+        rec = sum(size(t) for r in self.rec if r is not None for t in r if t is not None)
         return {"weights_gib": wbytes / gib, "kv_gib": kvb / gib, "state_gib": rec / gib, "kv_blocks": self.num_blocks,
                 "kv_tokens": self.num_blocks * BLOCK}

@@ -99,7 +99,7 @@ void token_shift(Tensor out, const Tensor& n32, const Tensor& carry, const Tenso
 void rope_cache_write(Tensor q, int64_t q_vecs, int64_t q_stride, int64_t q_off, const std::optional<Tensor>& q_out, int64_t q_cols,
                       Tensor kv, int64_t k_cols, int64_t k_vecs, int64_t k_stride, int64_t k_off, int64_t v_src, int64_t v_cols,
                       bool v_t, Tensor kcache, const std::optional<Tensor>& vcache, int64_t dims, bool interleaved, OptTensor cos_t, OptTensor sin_t,
-                      const Tensor& tok_pos, const Tensor& tok_seq, const Tensor& block_table) {
+                      const Tensor& tok_pos, const Tensor& tok_seq, const Tensor& block_table, OptTensor norm_w, double eps) {
   DLIA_ON_DEVICE_OF(kcache);
   check_fmat(q, "q"); check_fmat(kv, "kv"); check_act(kcache, "kcache");
   check_i32(tok_pos, "tok_pos"); check_i32(tok_seq, "tok_seq"); check_i32(block_table, "block_table");
@@ -110,6 +110,9 @@ void rope_cache_write(Tensor q, int64_t q_vecs, int64_t q_stride, int64_t q_off,
              "rope_cache_write: rotated q entries beyond the row");
   DLIA_CHECK(k_cols >= 1 && v_cols >= 0 && k_cols <= kv.size(1) && v_src >= 0 && v_src + v_cols <= kv.size(1) && k_off >= 0 &&
              (k_vecs == 0 || (k_vecs - 1) * k_stride + k_off + dims <= k_cols), "rope_cache_write: rotated k entries beyond the row");
+  const int64_t norm_cols = norm_w.has_value() ? norm_w->numel() : 0;
+  DLIA_CHECK(norm_cols <= k_cols && (norm_cols == 0 || k_vecs == 0 || dims == 0 || norm_cols <= k_off),
+             "rope_cache_write: the normed entries lead the k row, in front of the rotated ones");
   DLIA_CHECK(kcache.dim() == 4 && kcache.is_contiguous() && kcache.size(2) == 32, "rope_cache_write: kcache [blocks, G, 32, dk]");
   const int64_t G = kcache.size(1);
   DLIA_CHECK(G * kcache.size(3) == k_cols, "rope_cache_write: k row does not fill the cache row");
@@ -140,7 +143,28 @@ void rope_cache_write(Tensor q, int64_t q_vecs, int64_t q_stride, int64_t q_off,
                         kv.data_ptr<float>(), kv.stride(0), (int)k_cols, (int)k_vecs, (int)k_stride, (int)k_off, (int)v_src, (int)v_cols,
                         v_t ? 1 : 0, kcache.data_ptr(), vp, is_f32(kcache), (int)G, (int)dims, interleaved ? 1 : 0, cp, sp, table_pos,
                         tok_pos.data_ptr<int>(), tok_seq.data_ptr<int>(), block_table.data_ptr<int>(), (int)T, (int)block_table.size(1),
-                        (int)kcache.size(0), (int)block_table.size(0), cur_stream());
+                        (int)kcache.size(0), (int)block_table.size(0), opt_f32(norm_w, norm_cols, "norm_w"), (int)norm_cols, (float)eps, cur_stream());
+}
+
+// The queries alone: rotated in place and left in `q_out`'s type (a layer that reads another layer's cache rows).
+void rope_rows(Tensor q, int64_t q_vecs, int64_t q_stride, int64_t q_off, Tensor q_out, int64_t dims, bool interleaved, OptTensor cos_t,
+               OptTensor sin_t, const Tensor& tok_pos) {
+  DLIA_ON_DEVICE_OF(q);
+  check_fmat(q, "q"); check_act(q_out, "q_out"); check_mat(q_out, "q_out"); check_i32(tok_pos, "tok_pos");
+  const int64_t T = q_out.size(0), cols = q_out.size(1);
+  DLIA_CHECK(q.size(0) >= T && cols <= q.size(1) && tok_pos.numel() >= T, "rope_rows: rows");
+  DLIA_CHECK(dims >= 0 && dims % 2 == 0 && q_vecs >= 0 && q_stride >= 1 && q_off >= 0 &&
+             (q_vecs == 0 || (q_vecs - 1) * q_stride + q_off + dims <= q.size(1)), "rope_rows: rotation geometry");
+  const float *cp = nullptr, *sp = nullptr; int table_pos = 0;
+  if (dims > 0) {
+    DLIA_CHECK(cos_t.has_value() && sin_t.has_value(), "rope_rows: rotation needs its tables");
+    check_f32(*cos_t, "cos"); check_f32(*sin_t, "sin");
+    DLIA_CHECK(cos_t->dim() == 2 && cos_t->size(1) == dims / 2 && sin_t->sizes() == cos_t->sizes(), "rope_rows: tables [positions, dims / 2]");
+    cp = cos_t->data_ptr<float>(); sp = sin_t->data_ptr<float>(); table_pos = (int)cos_t->size(0);
+  }
+  dlia_rope_cache_write(q.data_ptr<float>(), q.stride(0), (int)q_vecs, (int)q_stride, (int)q_off, q_out.data_ptr(), q_out.stride(0), (int)cols,
+                        q.data_ptr<float>(), q.stride(0), 0, 0, 1, 0, 0, 0, 0, nullptr, nullptr, is_f32(q_out), 1, (int)dims, interleaved ? 1 : 0,
+                        cp, sp, table_pos, tok_pos.data_ptr<int>(), tok_pos.data_ptr<int>(), nullptr, (int)T, 0, 0, 0, nullptr, 0, 0.f, cur_stream());
 }
 
 // out [T, H * dv]; q [T, .] fp32, head h at columns h * q_head (maps * d entries); keys: rows of kcache [blocks, G, 32, k_row], map a
@@ -276,7 +300,8 @@ void gemm_blocks(Tensor out, const Tensor& x, const Tensor& w, OptTensor bias, i
 TORCH_LIBRARY_FRAGMENT(dlia, m) {
   m.def("par_norm(Tensor(a!)? out, Tensor(b!) out32, Tensor(c!) x, Tensor? ya, Tensor? yb, Tensor? ls1, Tensor? ls2, Tensor? w, Tensor(d!)? carry, Tensor tok_seq, float eps) -> ()");
   m.def("token_shift(Tensor(a!) out, Tensor n32, Tensor carry, Tensor mu, Tensor tok_pos, Tensor tok_seq) -> ()");
-  m.def("rope_cache_write(Tensor(a!) q, int q_vecs, int q_stride, int q_off, Tensor(b!)? q_out, int q_cols, Tensor(c!) kv, int k_cols, int k_vecs, int k_stride, int k_off, int v_src, int v_cols, bool v_t, Tensor(d!) kcache, Tensor(e!)? vcache, int dims, bool interleaved, Tensor? cos_t, Tensor? sin_t, Tensor tok_pos, Tensor tok_seq, Tensor block_table) -> ()");
+  m.def("rope_cache_write(Tensor(a!) q, int q_vecs, int q_stride, int q_off, Tensor(b!)? q_out, int q_cols, Tensor(c!) kv, int k_cols, int k_vecs, int k_stride, int k_off, int v_src, int v_cols, bool v_t, Tensor(d!) kcache, Tensor(e!)? vcache, int dims, bool interleaved, Tensor? cos_t, Tensor? sin_t, Tensor tok_pos, Tensor tok_seq, Tensor block_table, Tensor? norm_w=None, float eps=0.0) -> ()");
+  m.def("rope_rows(Tensor(a!) q, int q_vecs, int q_stride, int q_off, Tensor(b!) q_out, int dims, bool interleaved, Tensor? cos_t, Tensor? sin_t, Tensor tok_pos) -> ()");
   m.def("multi_attention(Tensor(a!) out, Tensor q, int q_head, Tensor kcache, Tensor vcache, int v_off, Tensor tok_pos, Tensor tok_seq, Tensor block_table, int H, int d, int dv, int maps, float scale, int window, int keep_first, float softcap, float lam, float post, float eps, Tensor? gate, int chunk=0, Tensor? sink=None) -> ()");
   m.def("tile_attention(Tensor(a!) out, Tensor q, int q_head, Tensor kcache, Tensor vt, Tensor q_start, Tensor ctx, Tensor slots, Tensor block_table, int max_q, int H, int d, int dv, int maps, float scale, int window, int keep_first, float softcap, float lam, float post, float eps, Tensor? gate, Tensor(b!)? part, int chunk=0, Tensor? sink=None) -> ()");
   m.def("tile_attention_part_floats(int B, int H, int G, int dv, int maps, int Gk=0) -> int");
@@ -291,6 +316,7 @@ TORCH_LIBRARY_IMPL(dlia, CUDA, m) {
   m.impl("par_norm", &par_norm);
   m.impl("token_shift", &token_shift);
   m.impl("rope_cache_write", &rope_cache_write);
+  m.impl("rope_rows", &rope_rows);
   m.impl("multi_attention", &multi_attention);
   m.impl("tile_attention", &tile_attention);
   m.impl("rglru_scan", &rglru_scan);

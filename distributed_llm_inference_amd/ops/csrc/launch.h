@@ -177,6 +177,10 @@ void dlia_moe_up(void* act, const void* x, const void* wg, const void* wu, int f
 void dlia_moe_down(float* y, const void* act, const void* wd, int f32, const int* tiles, const int* row_tok, int max_tiles, int wide,
                    int H, int F, long lda, int tile_rows, hipStream_t stream);
 // (wide: 128 / 256 output columns per workgroup, for steps with many rows; else 64)
+// desc [layers][8]: table offset, top, experts, offset of the tile list, of the row list, of the pair list, 128-row tiles allowed
+void dlia_moe_table_plan(int* tiles, int* row_tok, int* pair_row, const int* tables, const int* ids, const int* desc, int layers, int T,
+                         int vocab, int big_pairs, hipStream_t stream);
+void dlia_glu_act(void* act, int out_f32, long lda, const float* z, long ldz, int M, int F, float limit, int gated, hipStream_t stream);
 void dlia_moe_combine(float* out, const float* y, const int* pair_row, const float* wts, int T, int H, int top, long ldo,
                       const float* x, long ldx, hipStream_t stream);
 
@@ -192,7 +196,7 @@ void dlia_rope_cache_write(float* q, long ldq, int q_vecs, int q_stride, int q_o
                            long ldkv, int k_cols, int k_vecs, int k_stride, int k_off, int v_src, int v_cols, int v_t, void* kcache,
                            void* vcache, int f32, int G, int dims, int interleaved, const float* cos_t, const float* sin_t, int table_pos,
                            const int* tok_pos, const int* tok_seq, const int* block_table, int T, int max_blocks, int num_blocks,
-                           int table_rows, hipStream_t stream);
+                           int table_rows, const float* norm_w, int norm_cols, float eps, hipStream_t stream);
 void dlia_multi_attention(void* out, long ldo, const float* q, long ldq, int q_head, const void* kcache, int k_row,
                           const void* vcache, int v_row, int v_off, int f32, const int* tok_pos, const int* tok_seq,
                           const int* block_table, int T, int max_blocks, int num_blocks, int table_rows, int H, int G, int d, int dv,
@@ -233,6 +237,24 @@ int dlia_mixed_attention(void* out, long ldo, const void* q, long ldq, const voi
                          const int* q_start, const int* ctx, const int* slots, const int* block_table, int B, int max_q, int max_blocks,
                          int num_blocks, int table_rows, int H, int G, int d, int dv, int chunk, const float* sink, const float* gate,
                          long ldg, float* part, long part_floats, int T, hipStream_t stream);
+// ---- canon_ops.hip (convolved sublayer inputs, learned average over depth, PolyNorm) ----
+int dlia_stream_join_max_width(int vec);
+// Returns 1 (nothing launched) for rows wider than dlia_stream_join_max_width.
+int dlia_stream_join(void* out, int out_f32, long ldo, float* x, const float* x_in, const float* ya, long ldya, const float* yb, long ldyb,
+                     const float* ey, const int* pair_row, int top, float ew, float* hist, long hist_stride, int navg, const float* coef,
+                     const float* nw, float* rs, const float* close_w, float* close_carry, const float* taps, float* carry, int K,
+                     const int* tok_pos, const int* tok_seq, int T, int state_rows, int H, float eps, hipStream_t stream);
+void dlia_canon_conv(void* out, int out_f32, long ldo, const float* x, const float* rs, const float* nw, const float* taps,
+                     const float* carry, int K, const int* tok_pos, const int* tok_seq, int T, int state_rows, int H, hipStream_t stream);
+void dlia_poly_norm(void* out, int out_f32, long ldo, const float* z, long ldz, const float* coef, int T, int F, float eps,
+                    hipStream_t stream);
+// ---- linear_attention.hip (decays per head or per key channel, state in the slot, head norm and gate in the same call) ----
+long dlia_linear_attention_ws_floats(int rows, int B, int H, int d, int dv, int per_channel);
+int dlia_linear_attention(void* out, int out_f32, long ldo, const float* z, long ldz, float* state, const float* head_decay,
+                          const float* a2t, const float* a_b, int rank, const float* norm_w, const int* q_start, const int* ctx,
+                          const int* slots, int B, int T, int max_q, int H, int d, int dv, int state_rows, int col_q, int col_k,
+                          int col_v, int col_g, int col_a, float qscale, float inv_tau, float eps, float* ws, long ws_floats,
+                          hipStream_t stream);
 // ---- misc.hip -------------------------------------------------------------------------
 void dlia_advance_i32(int* x, int n, int delta, hipStream_t stream);
 void dlia_scatter_rows_i32(int* dst, const int* rows, const int* src, int nrows, int ncols, int dst_rows, hipStream_t stream);

@@ -11,6 +11,12 @@
 //                padded to whole 32-row tiles, and writes for every padded row its token (or -1), for every pair its row,
 //                for every tile its expert; tiles[0] holds the number of tiles. Rows of one expert are in no fixed order:
 //                every row is computed on its own, so the order does not reach the results.
+//   moe_table_plan  the same plan for every routed layer of a stack whose experts go by the token's id, in ONE launch ahead of the
+//                layers: workgroup l reads layer l's table [vocab, top] at the step's ids and lays out its pairs. Where the
+//                layers' parts lie in the shared buffers comes from a descriptor per layer (kPlanDesc numbers: table offset, top,
+//                experts, offset of the tile list, of the row list, of the pair list, whether 128-row tiles may be used).
+//   glu_act      the activation of one expert that runs for every token, from gate | up (| one more number, whose sigmoid
+//                multiplies the row) in fp32
 //   moe_up       grid (column blocks, tiles): act[row, f] = g s(1.702 g) (u + 1), g = min(x . Wg[e][f], limit),
 //                u = clamp(x . Wu[e][f], -limit, limit), x the row's token; with limit <= 0 the plain silu(g) * u.
 //                Gate and up accumulate over the same A fragments.
@@ -92,16 +98,18 @@ __global__ __launch_bounds__(64) void moe_route_kernel(int* __restrict__ sel, fl
   for (int r = 0; r < top; ++r) wts[(long)t * top + r] *= inv;
 }
 
-// tiles: [0] number of tiles, [1 + i] expert of tile i. row_tok [max_rows], pair_row [T * top].
-__global__ __launch_bounds__(1024) void moe_plan_kernel(int* __restrict__ tiles, int* __restrict__ row_tok,
-                                                        int* __restrict__ pair_row, const int* __restrict__ sel, int pairs,
-                                                        int top, int E, int max_rows, int tile_rows) {
-  __shared__ int count[kMoeMaxExperts], start[kMoeMaxExperts], fill[kMoeMaxExperts];
-  __shared__ int ntiles;
+// Lays out the pairs of one layer. expert(i): the expert of pair i (i / top is its token). 1024 threads.
+// tiles: [0] number of tiles, [1 + i] expert of tile i. row_tok [max_rows], pair_row [pairs].
+template <typename Sel>
+__device__ __forceinline__ void plan_pairs(int* __restrict__ tiles, int* __restrict__ row_tok, int* __restrict__ pair_row, int pairs,
+                                           int top, int E, int max_rows, int tile_rows, int* count, int* start, int* fill, int* ntiles,
+                                           Sel expert) {
   for (int e = threadIdx.x; e < E; e += 1024) { count[e] = 0; fill[e] = 0; }
   __syncthreads();
-  for (int i = threadIdx.x; i < pairs; i += 1024)
-    if (sel[i] < E) atomicAdd(&count[sel[i]], 1);
+  for (int i = threadIdx.x; i < pairs; i += 1024) {
+    const int e = expert(i);
+    if (e < E) atomicAdd(&count[e], 1);
+  }
   __syncthreads();
   if (threadIdx.x == 0) {
     int at = 0, nt = 0;
@@ -112,18 +120,60 @@ __global__ __launch_bounds__(1024) void moe_plan_kernel(int* __restrict__ tiles,
       nt += n; at += n * tile_rows;
     }
     tiles[0] = nt;
-    ntiles = nt;
+    *ntiles = nt;
   }
   __syncthreads();
-  const int used = ntiles * tile_rows;
+  const int used = *ntiles * tile_rows;
   for (int i = threadIdx.x; i < max_rows; i += 1024) row_tok[i] = -1;
   __syncthreads();
   for (int i = threadIdx.x; i < pairs; i += 1024) {
-    const int e = sel[i];
+    const int e = expert(i);
     if (e >= E) { pair_row[i] = -1; continue; }                      // (an identity expert: no row)
     const int r = start[e] + atomicAdd(&fill[e], 1);
     if (r < max_rows && r < used) { row_tok[r] = i / top; pair_row[i] = r; }
   }
+}
+
+__global__ __launch_bounds__(1024) void moe_plan_kernel(int* __restrict__ tiles, int* __restrict__ row_tok,
+                                                        int* __restrict__ pair_row, const int* __restrict__ sel, int pairs,
+                                                        int top, int E, int max_rows, int tile_rows) {
+  __shared__ int count[kMoeMaxExperts], start[kMoeMaxExperts], fill[kMoeMaxExperts];
+  __shared__ int ntiles;
+  plan_pairs(tiles, row_tok, pair_row, pairs, top, E, max_rows, tile_rows, count, start, fill, &ntiles, [&](int i) { return sel[i]; });
+}
+
+constexpr int kPlanDesc = 8;
+constexpr int kTableMaxExperts = 1024;
+
+__global__ __launch_bounds__(1024) void moe_table_plan_kernel(int* __restrict__ tiles, int* __restrict__ row_tok,
+                                                              int* __restrict__ pair_row, const int* __restrict__ tables,
+                                                              const int* __restrict__ ids, const int* __restrict__ desc, int T, int vocab,
+                                                              int big_pairs) {
+  __shared__ int count[kTableMaxExperts], start[kTableMaxExperts], fill[kTableMaxExperts];
+  __shared__ int ntiles;
+  const int* d = desc + blockIdx.x * kPlanDesc;
+  const int* table = tables + d[0];
+  const int top = d[1], E = d[2], pairs = T * top;
+  const int tile_rows = d[6] && pairs >= big_pairs ? kMoeBigRows : kMoeRows;
+  plan_pairs(tiles + d[3], row_tok + d[4], pair_row + d[5], pairs, top, E, ((pairs + tile_rows - 1) / tile_rows + E) * tile_rows, tile_rows,
+             count, start, fill, &ntiles, [&](int i) {
+               int id = ids[i / top];
+               id = id < 0 ? 0 : (id >= vocab ? vocab - 1 : id);     // (as the embedding does: never fault on a bad id)
+               const int e = table[(long)id * top + i % top];
+               return e < 0 ? 0 : e;
+             });
+}
+
+template <typename OT>
+__global__ __launch_bounds__(256) void glu_act_kernel(OT* __restrict__ act, long lda, const float* __restrict__ z, long ldz, int F,
+                                                      float limit, int gated) {
+  const long m = blockIdx.y;
+  const int c = blockIdx.x * 256 + threadIdx.x;
+  if (c >= F) return;
+  const float* zr = z + m * ldz;
+  float v = expert_act(zr[c], zr[F + c], limit);
+  if (gated) v *= 1.f / (1.f + expf(-zr[2 * F]));
+  act[m * lda + c] = (OT)v;
 }
 
 // Row tiles of the plan: 32 rows. A workgroup of four waves covers one row tile by 128 (up) or 256 (down) output columns; a
@@ -434,4 +484,18 @@ extern "C" void dlia_moe_combine(float* out, const float* y, const int* pair_row
                                  const float* x, long ldx, hipStream_t stream) {
   if (T <= 0) return;
   hipLaunchKernelGGL(dlia::moe_combine_kernel, dim3(T), dim3(256), 0, stream, out, y, pair_row, wts, H, top, ldo, x, ldx);
+}
+
+extern "C" void dlia_moe_table_plan(int* tiles, int* row_tok, int* pair_row, const int* tables, const int* ids, const int* desc, int layers,
+                                    int T, int vocab, int big_pairs, hipStream_t stream) {
+  if (layers <= 0) return;
+  hipLaunchKernelGGL(dlia::moe_table_plan_kernel, dim3(layers), dim3(1024), 0, stream, tiles, row_tok, pair_row, tables, ids, desc, T, vocab,
+                     big_pairs);
+}
+
+extern "C" void dlia_glu_act(void* act, int out_f32, long lda, const float* z, long ldz, int M, int F, float limit, int gated, hipStream_t stream) {
+  if (M <= 0 || F <= 0) return;
+  const dim3 grid((F + 255) / 256, M);
+  if (out_f32) hipLaunchKernelGGL(dlia::glu_act_kernel<float>, grid, dim3(256), 0, stream, (float*)act, lda, z, ldz, F, limit, gated);
+  else hipLaunchKernelGGL(dlia::glu_act_kernel<dlia::bf16>, grid, dim3(256), 0, stream, (dlia::bf16*)act, lda, z, ldz, F, limit, gated);
 }

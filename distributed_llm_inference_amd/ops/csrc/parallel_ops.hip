@@ -10,7 +10,8 @@
 //                   start of a portion, zeros at position 0
 //   rope_cache_write per token: rotates the first `dims` entries of a set of q vectors and of the k vectors (pairs
 //                   (2i, 2i + 1) or (i, i + dims / 2), angles from a table by position), optionally leaves q in the
-//                   GEMMs' input type, and writes the k row (and the v row) into the paged cache
+//                   GEMMs' input type, and writes the k row (and the v row) into the paged cache; the first entries of
+//                   the k row may be RMS-normed with a weight on the way (a latent), or there may be no k row at all
 //   multi_attention one wave per (token, head): softmax attention over the paged cache with a window that also keeps
 //                   the sequence's first tokens, scores through cap tanh(s / cap); with two maps per head both are
 //                   walked at once over the shared values and combined as rms(a1 - lam a2) (1 - diff) sigmoid(gate).
@@ -112,11 +113,19 @@ __global__ __launch_bounds__(kParThreads) void rope_cache_write_kernel(
     T* __restrict__ kcache, T* __restrict__ vcache, int G, int dims, int interleaved, const float* __restrict__ cos_t,
     const float* __restrict__ sin_t,
     int table_pos, const int* __restrict__ tok_pos, const int* __restrict__ tok_seq, const int* __restrict__ block_table,
-    int max_blocks, int num_blocks, int table_rows) {
+    int max_blocks, int num_blocks, int table_rows, const float* __restrict__ norm_w, int norm_cols, float eps) {
+  __shared__ float scratch[16];
   const int t = blockIdx.x;
   const int pos = tok_pos[t], slot = tok_seq[t];
   float* qrow = q + (long)t * ldq;
   float* krow = kv + (long)t * ldkv;
+  if (norm_w) {            // the first norm_cols entries of the k row are RMS-normed (they are not among the rotated ones)
+    float s = 0.f;
+    for (int i = threadIdx.x; i < norm_cols; i += kParThreads) { const float v = krow[i]; s += v * v; }
+    s = block_sum(s, scratch);
+    const float r = 1.f / sqrtf(s / norm_cols + eps);
+    for (int i = threadIdx.x; i < norm_cols; i += kParThreads) krow[i] *= r * norm_w[i];
+  }
   if (dims > 0 && pos >= 0 && pos < table_pos) {
     const float* cs = cos_t + (long)pos * (dims >> 1);
     const float* sn = sin_t + (long)pos * (dims >> 1);
@@ -126,6 +135,7 @@ __global__ __launch_bounds__(kParThreads) void rope_cache_write_kernel(
   __syncthreads();
   if (q_out)
     for (int i = threadIdx.x; i < q_cols; i += kParThreads) q_out[(long)t * ldqo + i] = (T)qrow[i];
+  if (!kcache) return;     // (queries alone: the layer reads another layer's rows)
   int blk = -1;
   if (slot >= 0 && slot < table_rows && pos >= 0 && pos / kParBlock < max_blocks) blk = block_table[(long)slot * max_blocks + pos / kParBlock];
   if (blk < 0 || blk >= num_blocks) return;
@@ -777,18 +787,18 @@ extern "C" void dlia_rope_cache_write(float* q, long ldq, int q_vecs, int q_stri
                                       int v_t, void* kcache, void* vcache, int f32, int G, int dims, int interleaved, const float* cos_t,
                                       const float* sin_t, int table_pos, const int* tok_pos, const int* tok_seq,
                                       const int* block_table, int T, int max_blocks, int num_blocks, int table_rows,
-                                      hipStream_t stream) {
+                                      const float* norm_w, int norm_cols, float eps, hipStream_t stream) {
   if (T <= 0) return;
   if (f32)
     hipLaunchKernelGGL(rope_cache_write_kernel<float>, dim3(T), dim3(kParThreads), 0, stream, q, ldq, q_vecs, q_stride, q_off,
                        (float*)q_out, ldqo, q_cols, kv, ldkv, k_cols, k_vecs, k_stride, k_off, v_src, v_cols, v_t, (float*)kcache,
                        (float*)vcache, G, dims, interleaved, cos_t, sin_t, table_pos, tok_pos, tok_seq, block_table, max_blocks,
-                       num_blocks, table_rows);
+                       num_blocks, table_rows, norm_w, norm_cols, eps);
   else
     hipLaunchKernelGGL(rope_cache_write_kernel<bf16>, dim3(T), dim3(kParThreads), 0, stream, q, ldq, q_vecs, q_stride, q_off,
                        (bf16*)q_out, ldqo, q_cols, kv, ldkv, k_cols, k_vecs, k_stride, k_off, v_src, v_cols, v_t, (bf16*)kcache,
                        (bf16*)vcache, G, dims, interleaved, cos_t, sin_t, table_pos, tok_pos, tok_seq, block_table, max_blocks,
-                       num_blocks, table_rows);
+                       num_blocks, table_rows, norm_w, norm_cols, eps);
 }
 
 template <typename T, typename OT>
