@@ -1,7 +1,8 @@
 """Prefill and decode throughput of a Letarax stack beside a Llama stack of equal size (`bench.py --hybrid-compare`), of a
 Nufapel stack beside the Letarax stack of equal size (`bench.py --gated-compare`), of a Tezesun stack beside the
-Letarax stack of equal size (`bench.py --parallel-compare`), and of a Zovozen stack beside the Nufapel stack of equal size
-(`bench.py --postnorm-compare`).
+Letarax stack of equal size (`bench.py --parallel-compare`), of a Zovozen stack beside the Nufapel stack of equal size
+(`bench.py --postnorm-compare`), and of a Pifutar stack beside the Nufapel and the Tezesun stack of equal size
+(`bench.py --canon-compare`).
 
 Both models get random weights and the same width, head counts, head size, feed-forward width, depth and
 vocabulary; the Letarax stack has three attention layers (windowed, with the sink and value mixing) to one delta-rule
@@ -44,6 +45,14 @@ def postnorm_specs(name: str):
     depth: the Nufapel stack (attention beside a matrix memory in three layers of four, routed feed-forwards)."""
     from distributed_llm_inference_amd.models.spec import BUILTIN_SPECS
     return BUILTIN_SPECS[f"zovozen-{name}"], BUILTIN_SPECS[f"nufapel-{name}"]
+
+
+def canon_specs(name: str):
+    """The Pifutar stack of a size (retention, gated linear attention, latent attention with a window, a layer that reads its rows;
+    one dense layer in four, the others routed by token id with a shared expert) beside the two existing designs that share its
+    mechanisms: Nufapel (matrix states in the slots, routed feed-forwards) and Tezesun (latent attention, dense feed-forwards)."""
+    from distributed_llm_inference_amd.models.spec import BUILTIN_SPECS
+    return tuple(BUILTIN_SPECS[f"{f}-{name}"] for f in ("pifutar", "nufapel", "tezesun"))
 
 
 def specs(name: str):
@@ -110,15 +119,18 @@ def time_decode(ex, rows: int, ctx: int, iters: int) -> float:
     return e0.elapsed_time(e1) / 1e3 / iters
 
 
-def main(sizes=None, iters: int = 8, out=sys.stdout, gated: bool = False, parallel: bool = False, postnorm: bool = False) -> int:
+def main(sizes=None, iters: int = 8, out=sys.stdout, gated: bool = False, parallel: bool = False, postnorm: bool = False,
+         canon: bool = False) -> int:
     import gc
     import torch
     rows, ctx, plen = 64, 1024, 2048
     for name in (sizes or list(SIZES)):
-        rec = {"metric": "zovozen_vs_nufapel_tokens_per_s" if postnorm else "tezesun_vs_letarax_tokens_per_s" if parallel else "nufapel_vs_letarax_tokens_per_s" if gated else "letarax_vs_llama_tokens_per_s", "size": name, "dtype": "bf16", "data": "synthetic", "weights": "random",
+        pair = canon_specs(name) if canon else postnorm_specs(name) if postnorm else parallel_specs(name) if parallel else gated_specs(name) if gated else specs(name)
+        new, *old = [x.family for x in pair]
+        rec = {"metric": f"{new}_vs_{'_'.join(old)}_tokens_per_s", "size": name, "dtype": "bf16", "data": "synthetic", "weights": "random",
                "config": dict(zip(("width", "heads", "kv_heads", "head_dim", "ff", "layers", "window"), SIZES[name])),
                "prefill": {"prompts": 1, "tokens": plen}, "decode": {"rows": rows, "context": ctx}}
-        for spec in (postnorm_specs(name) if postnorm else parallel_specs(name) if parallel else gated_specs(name) if gated else specs(name)):
+        for spec in pair:
             t0 = time.perf_counter()
             ex = build(spec, rows, plen, max(plen, ctx + 256))
             tp = time_prefill(ex, 1, plen, iters)
@@ -132,9 +144,9 @@ def main(sizes=None, iters: int = 8, out=sys.stdout, gated: bool = False, parall
             del ex
             gc.collect()
             torch.cuda.empty_cache()
-        new, old = ("zovozen", "nufapel") if postnorm else ("tezesun", "letarax") if parallel else ("nufapel", "letarax") if gated else ("letarax", "llama")
-        rec["prefill_ratio"] = round(rec[new]["prefill_tok_s"] / rec[old]["prefill_tok_s"], 3)
-        rec["decode_ratio"] = round(rec[new]["decode_tok_s"] / rec[old]["decode_tok_s"], 3)
+        for i, o in enumerate(old):
+            for what in ("prefill", "decode"):
+                rec[f"{what}_ratio" if i == 0 else f"{what}_ratio_{o}"] = round(rec[new][f"{what}_tok_s"] / rec[o][f"{what}_tok_s"], 3)
         out.write(json.dumps(rec) + "\n")
         out.flush()
     return 0
