@@ -151,6 +151,8 @@ class HybridGpuStage(GpuStage):
         # the any-shape kernel. DLIA_HYBRID_PACKED=0 keeps everything on the any-shape kernel (A/B).
         self._packed = dtype == "bf16" and os.environ.get("DLIA_HYBRID_PACKED", "1") != "0"
         self.decode_rows = 256
+        # latent attention in bf16: DLIA_LATENT_ATTN=0 keeps it on the general tile kernel (A/B)
+        self._latent_fast = os.environ.get("DLIA_LATENT_ATTN", "1") != "0"
         self._shapes = []                        # (N, K, has_bias) of every packed GEMM, for the workspace
         # Attention layers whose keys and values have one size, 64 or 128, with up to 16 query heads per key / value head run
         # on the library's MFMA attention kernels (fragment-ordered cache, the windowed / sink instantiations), bf16 only;
@@ -759,6 +761,22 @@ class HybridGpuStage(GpuStage):
             return ls.kv_rank + ls.rot_dim, ls.kv_rank if self._tile[li] else 0
         return ls.kv_heads * ls.maps * ls.dim, ls.kv_heads * ls.vdim
 
+    def _latent_attention(self, olat, qa16, kc, vc, q_start, ctx, slots, max_q: int, ls, part):
+        """Attention of all heads over the layer's cached rows (bf16, matrix cores): the kernel made for one shared row where the sizes
+        come in whole 16-byte pieces, the general tile kernel otherwise."""
+        D, R = ls.kv_rank + ls.rot_dim, ls.kv_rank
+        if self._latent_fast and self.K.latent_attention_fits(D, R):
+            self.K.latent_attention(olat, qa16, kc, vc, q_start, ctx, slots, self.block_table, max_q, ls.heads, ls.scale, ls.window or 0, part)
+        else:
+            self.K.tile_attention(olat, qa16, D, kc, vc, q_start, ctx, slots, self.block_table, max_q, ls.heads, D, R, 1, ls.scale, ls.window or 0, 0,
+                                  0.0, 0.0, 1.0, self.spec.norm_eps, None, part)
+
+    def _latent_part_floats(self, rows: int, B: int, ls) -> int:
+        """Workspace of `_latent_attention`'s key splits for steps of up to `rows` tokens in up to B sequences."""
+        D, R = ls.kv_rank + ls.rot_dim, ls.kv_rank
+        n = max(int(self.K.tile_attention_part_floats(b, ls.heads, 1, R, 1)) for b in range(1, B + 1))
+        return max(n, int(self.K.latent_attention_part_floats(rows, B, ls.heads, R))) if self._latent_fast and self.K.latent_attention_fits(D, R) else n
+
     def _load_par(self, weights: StageWeights, f32, mat):
         """Device weights of a stack with parallel layers. A mixer's input projections are ONE matrix; what a recurrence or a
         score needs in fp32 (gate matrices, decay rates, norm weights, rotation tables) stays fp32 in both modes."""
@@ -840,9 +858,10 @@ class HybridGpuStage(GpuStage):
                     ws_floats = max([ws_floats] + [int(self.K.gemm_ws_floats(m_, n_, k_)) for n_, k_, _ in self._shapes])
         part = 1                  # partial results of the key splits of single-token steps (any number of rows up to B)
         for ls, tile in zip(self.specs, self._tile):
-            if tile:
-                dv = ls.kv_rank if ls.kind == "latent_attention" else ls.vdim
-                part = max([part] + [int(self.K.tile_attention_part_floats(b_, ls.heads, ls.kv_heads, dv, ls.maps)) for b_ in range(1, B + 1)])
+            if tile and ls.kind == "latent_attention":
+                part = max(part, self._latent_part_floats(rows, B, ls))
+            elif tile:
+                part = max([part] + [int(self.K.tile_attention_part_floats(b_, ls.heads, ls.kv_heads, ls.vdim, ls.maps)) for b_ in range(1, B + 1)])
         scan = max([1] + [int(self.K.rglru_scan_ws_floats(rows, B, ls.rec_width)) for ls in self.specs if ls.kind == "rglru"])
         return SimpleNamespace(
             part=z(part), scan_ws=z(scan),
@@ -903,8 +922,7 @@ class HybridGpuStage(GpuStage):
                 if tile:
                     qa16 = view(wk.qa16, Hh * (R + dr))
                     K.gemm_blocks(qa16, q16, p["w_abs"], None, d + dr, R + dr)
-                    K.tile_attention(olat, qa16, R + dr, kc, vc, q_start, ctx, slots, table, max_q, Hh, R + dr, R, 1, ls.scale, 0, 0, 0.0,
-                                     0.0, 1.0, eps, None, wk.part)
+                    self._latent_attention(olat, qa16, kc, vc, q_start, ctx, slots, max_q, ls, wk.part)
                 else:
                     K.gemm_blocks(qa, q16, p["w_abs"], None, d + dr, R + dr)
                     K.multi_attention(olat, qa, R + dr, kc, kc, 0, tok_pos, tok_seq, table, Hh, R + dr, R, 1, ls.scale, 0, 0, 0.0, 0.0, 1.0,
@@ -1215,8 +1233,8 @@ class HybridGpuStage(GpuStage):
                     lin = max(lin, int(self.K.linear_attention_ws_floats(rows, B, ls.heads, ls.dim, ls.vdim, not ls.head_decay)))
             else:
                 q16, qa, ol = max(q16, ls.heads * (ls.dim + ls.rot_dim)), max(qa, ls.heads * (ls.kv_rank + ls.rot_dim)), max(ol, ls.heads * ls.kv_rank)
-                if tile:          # (key splits of single-token steps, of any number of rows up to B)
-                    part = max([part] + [int(self.K.tile_attention_part_floats(b_, ls.heads, 1, ls.kv_rank, 1)) for b_ in range(1, B + 1)])
+                if tile:
+                    part = max(part, self._latent_part_floats(rows, B, ls))
             if ls.moe is not None:
                 e = ls.moe
                 for t in {rows, min(rows, (self.BIG_PAIRS - 1) // e.top)}:      # (the most rows of either tile size)
@@ -1299,8 +1317,7 @@ class HybridGpuStage(GpuStage):
                 if tile:
                     qa16 = view(wk.qa16, Hh * (R + dr))
                     K.gemm_blocks(qa16, q16, p["w_abs"], None, d + dr, R + dr)
-                    K.tile_attention(olat, qa16, R + dr, kc, vc, q_start, ctx, slots, table, max_q, Hh, R + dr, R, 1, ls.scale, ls.window or 0, 0,
-                                     0.0, 0.0, 1.0, eps, None, wk.part)
+                    self._latent_attention(olat, qa16, kc, vc, q_start, ctx, slots, max_q, ls, wk.part)
                 else:
                     qa = view(wk.qa, Hh * (R + dr))
                     K.gemm_blocks(qa, q16, p["w_abs"], None, d + dr, R + dr)

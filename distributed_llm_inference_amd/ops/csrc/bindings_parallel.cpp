@@ -241,6 +241,36 @@ void tile_attention(Tensor out, const Tensor& q, int64_t q_head, const Tensor& k
   DLIA_CHECK(rc == 0, "tile_attention: sizes must be multiples of 8 (d, key row, q head stride, q row), maps * d <= 1024, dv <= 512");
 }
 
+// Attention over one cached row per token whose first R entries are the values: q [T, H D] and out [T, H R] bf16, contiguous; kcache
+// [blocks, 1, 32, D], vt [blocks, 1, R, 32]; window 0: the whole context.
+void latent_attention(Tensor out, const Tensor& q, const Tensor& kcache, const Tensor& vt, const Tensor& q_start, const Tensor& ctx,
+                      const Tensor& slots, const Tensor& block_table, int64_t max_q, int64_t H, double scale, int64_t window,
+                      const std::optional<Tensor>& part) {
+  DLIA_ON_DEVICE_OF(out);
+  check_i32(q_start, "q_start"); check_i32(ctx, "ctx"); check_i32(slots, "slots"); check_i32(block_table, "block_table");
+  for (const Tensor* t : std::initializer_list<const Tensor*>{&out, &q, &kcache, &vt})
+    DLIA_CHECK(t->is_cuda() && t->scalar_type() == at::kBFloat16 && t->is_contiguous() && reinterpret_cast<uintptr_t>(t->data_ptr()) % 16 == 0,
+               "latent_attention: contiguous bfloat16 on the GPU");
+  const int64_t T = out.size(0), B = ctx.numel();
+  DLIA_CHECK(kcache.dim() == 4 && vt.dim() == 4 && kcache.size(1) == 1 && vt.size(1) == 1 && kcache.size(2) == 32 && vt.size(3) == 32 &&
+             kcache.size(0) == vt.size(0) && kcache.size(0) >= 1, "latent_attention: kcache [blocks, 1, 32, D], vt [blocks, 1, R, 32]");
+  const int64_t D = kcache.size(3), R = vt.size(2);
+  DLIA_CHECK(H >= 1 && out.dim() == 2 && q.dim() == 2 && out.size(1) == H * R && q.size(0) >= T && q.size(1) == H * D, "latent_attention: q [T, H D], out [T, H R]");
+  DLIA_CHECK(q_start.numel() >= B + 1 && slots.numel() >= B && block_table.dim() == 2 && block_table.size(1) >= 1 && max_q >= 0 && max_q <= T && window >= 0,
+             "latent_attention: metadata");
+  float* pp = nullptr; long pn = 0;
+  if (part.has_value()) { check_f32(*part, "part"); pp = part->data_ptr<float>(); pn = part->numel(); }
+  const int rc = dlia_latent_attention(out.data_ptr(), q.data_ptr(), kcache.data_ptr(), vt.data_ptr(), q_start.data_ptr<int>(), ctx.data_ptr<int>(),
+                                       slots.data_ptr<int>(), block_table.data_ptr<int>(), (int)B, (int)T, (int)max_q, (int)block_table.size(1),
+                                       (int)kcache.size(0), (int)block_table.size(0), (int)H, (int)D, (int)R, (float)scale, (int)window, pp, pn, cur_stream());
+  DLIA_CHECK(rc == 0, "latent_attention: rows of ", D, " entries with ", R, " values are not taken (latent_attention_fits)");
+}
+
+bool latent_attention_fits(int64_t D, int64_t R) { return dlia_latent_attention_fits((int)D, (int)R) != 0; }
+int64_t latent_attention_part_floats(int64_t rows, int64_t B, int64_t H, int64_t R) {
+  return dlia_latent_attention_part_floats((int)rows, (int)B, (int)H, (int)R);
+}
+
 int64_t rglru_scan_ws_floats(int64_t rows, int64_t B, int64_t W) { return dlia_rglru_scan_ws_floats((int)rows, (int)B, (int)W); }
 
 int64_t tile_attention_part_floats(int64_t B, int64_t H, int64_t G, int64_t dv, int64_t maps, int64_t Gk) {
@@ -304,6 +334,9 @@ TORCH_LIBRARY_FRAGMENT(dlia, m) {
   m.def("rope_rows(Tensor(a!) q, int q_vecs, int q_stride, int q_off, Tensor(b!) q_out, int dims, bool interleaved, Tensor? cos_t, Tensor? sin_t, Tensor tok_pos) -> ()");
   m.def("multi_attention(Tensor(a!) out, Tensor q, int q_head, Tensor kcache, Tensor vcache, int v_off, Tensor tok_pos, Tensor tok_seq, Tensor block_table, int H, int d, int dv, int maps, float scale, int window, int keep_first, float softcap, float lam, float post, float eps, Tensor? gate, int chunk=0, Tensor? sink=None) -> ()");
   m.def("tile_attention(Tensor(a!) out, Tensor q, int q_head, Tensor kcache, Tensor vt, Tensor q_start, Tensor ctx, Tensor slots, Tensor block_table, int max_q, int H, int d, int dv, int maps, float scale, int window, int keep_first, float softcap, float lam, float post, float eps, Tensor? gate, Tensor(b!)? part, int chunk=0, Tensor? sink=None) -> ()");
+  m.def("latent_attention(Tensor(a!) out, Tensor q, Tensor kcache, Tensor vt, Tensor q_start, Tensor ctx, Tensor slots, Tensor block_table, int max_q, int H, float scale, int window, Tensor(b!)? part) -> ()");
+  m.def("latent_attention_fits(int D, int R) -> bool");
+  m.def("latent_attention_part_floats(int rows, int B, int H, int R) -> int");
   m.def("tile_attention_part_floats(int B, int H, int G, int dv, int maps, int Gk=0) -> int");
   m.def("rglru_scan(Tensor(a!) out, Tensor u, Tensor gates, Tensor ypre, Tensor clam, Tensor(b!) state, Tensor q_start, Tensor ctx, Tensor slots, int bw, int max_q, Tensor(c!)? ws) -> ()");
   m.def("rglru_scan_ws_floats(int rows, int B, int W) -> int");
@@ -318,6 +351,7 @@ TORCH_LIBRARY_IMPL(dlia, CUDA, m) {
   m.impl("rope_cache_write", &rope_cache_write);
   m.impl("rope_rows", &rope_rows);
   m.impl("multi_attention", &multi_attention);
+  m.impl("latent_attention", &latent_attention);
   m.impl("tile_attention", &tile_attention);
   m.impl("rglru_scan", &rglru_scan);
   m.impl("xielu", &xielu);
@@ -326,6 +360,8 @@ TORCH_LIBRARY_IMPL(dlia, CUDA, m) {
 }
 
 TORCH_LIBRARY_IMPL(dlia, CompositeExplicitAutograd, m) {
+  m.impl("latent_attention_fits", &latent_attention_fits);
+  m.impl("latent_attention_part_floats", &latent_attention_part_floats);
   m.impl("tile_attention_part_floats", &tile_attention_part_floats);
   m.impl("rglru_scan_ws_floats", &rglru_scan_ws_floats);
 }

@@ -255,6 +255,12 @@ int dlia_linear_attention(void* out, int out_f32, long ldo, const float* z, long
                           const int* slots, int B, int T, int max_q, int H, int d, int dv, int state_rows, int col_q, int col_k,
                           int col_v, int col_g, int col_a, float qscale, float inv_tau, float eps, float* ws, long ws_floats,
                           hipStream_t stream);
+// ---- latent_attention.hip (many query heads over one cached row per token, bf16, matrix cores) ----
+int dlia_latent_attention_fits(int D, int R);
+long dlia_latent_attention_part_floats(int rows, int B, int H, int R);
+int dlia_latent_attention(void* out, const void* q, const void* kcache, const void* vt, const int* q_start, const int* ctx, const int* slots,
+                          const int* block_table, int B, int T, int max_q, int max_blocks, int num_blocks, int table_rows, int H, int D,
+                          int R, float scale, int window, float* part, long part_floats, hipStream_t stream);
 // ---- misc.hip -------------------------------------------------------------------------
 void dlia_advance_i32(int* x, int n, int delta, hipStream_t stream);
 void dlia_scatter_rows_i32(int* dst, const int* rows, const int* src, int nrows, int ncols, int dst_rows, hipStream_t stream);
