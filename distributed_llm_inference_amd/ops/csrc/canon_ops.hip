@@ -85,11 +85,19 @@ __global__ __launch_bounds__(kCanonThreads) void stream_join_kernel(
       Unit<V> s;
 #pragma unroll
       for (int e = 0; e < V; ++e) s.v[e] = 0.f;
-      for (int j = 0; j < navg; ++j) {
-        const Unit<V> a = ldu<V>(hist + (long)j * hist_stride + row + c);
-        const float cj = coef[j];
+      for (int j0 = 0; j0 < navg; j0 += 4) {           // (four rows in flight)
+        Unit<V> a[4]; float cj[4];
 #pragma unroll
-        for (int e = 0; e < V; ++e) s.v[e] += cj * a.v[e];
+        for (int j = 0; j < 4; ++j) {
+          const int jj = min(j0 + j, navg - 1);
+          a[j] = ldu<V>(hist + (long)jj * hist_stride + row + c);
+          cj[j] = j0 + j < navg ? coef[jj] : 0.f;
+        }
+#pragma unroll
+        for (int j = 0; j < 4; ++j)
+          if (j0 + j < navg)
+#pragma unroll
+            for (int e = 0; e < V; ++e) s.v[e] += cj[j] * a[j].v[e];
       }
       const float cl = coef[navg];
 #pragma unroll
@@ -140,10 +148,11 @@ __global__ __launch_bounds__(kCanonThreads) void stream_join_kernel(
   }
 }
 
-// A workgroup takes kConvRows consecutive tokens by 256 units of V channels.
+// A workgroup takes kConvRows consecutive tokens by 256 units of V channels and slides the last h over them in registers: a row is
+// read once per tile (and the K - 1 rows in front of it). KT: taps known at compile time, 0: any number, every row read again.
 constexpr int kConvRows = 8;
 
-template <typename OT, int V>
+template <typename OT, int V, int KT>
 __global__ __launch_bounds__(kCanonThreads) void canon_conv_kernel(
     OT* __restrict__ out, long ldo, const float* __restrict__ x, const float* __restrict__ rs, const float* __restrict__ nw,
     const float* __restrict__ taps, const float* __restrict__ carry, int K, const int* __restrict__ tok_pos,
@@ -153,34 +162,57 @@ __global__ __launch_bounds__(kCanonThreads) void canon_conv_kernel(
   Unit<V> w = ldu<V>(nw + c);
 #pragma unroll
   for (int e = 0; e < V; ++e) w.v[e] += 1.f;
-  const int t1 = min(T, ((int)blockIdx.x + 1) * kConvRows);
-  for (int t = blockIdx.x * kConvRows; t < t1; ++t) {
-    const int slot = tok_seq[t], pos = tok_pos[t];
+  auto row_h = [&](int t) {
+    Unit<V> h = ldu<V>(x + (long)t * H + c);
     const float f = rs[t];
-    const Unit<V> xt = ldu<V>(x + (long)t * H + c);
-    Unit<V> h, g;
 #pragma unroll
-    for (int e = 0; e < V; ++e) h.v[e] = xt.v[e] * f * w.v[e];
-    g = h;
-    if (taps) {
-      Unit<V> s;
+    for (int e = 0; e < V; ++e) h.v[e] = h.v[e] * f * w.v[e];
+    return h;
+  };
+  // h of the token `back` places before token t of the step (position pos of the sequence in `slot`); zeros in front of the sequence
+  auto earlier = [&](int t, int back, int slot, int pos) {
+    const int p = pos - back;
+    Unit<V> h;
 #pragma unroll
-      for (int e = 0; e < V; ++e) s.v[e] = 0.f;
+    for (int e = 0; e < V; ++e) h.v[e] = 0.f;
+    if (p < 0) return h;
+    if (t - back >= 0 && tok_seq[t - back] == slot && tok_pos[t - back] == p) return row_h(t - back);
+    if (slot >= 0 && slot < state_rows) return ldu<V>(carry + ((long)slot * (K - 1) + p % (K - 1)) * H + c);
+    return h;
+  };
+  constexpr int KR = KT > 1 ? KT : 1;
+  Unit<V> tap[KR], win[KR];                            // win[j]: the h that meets tap j (the last one is the token's own)
+  if constexpr (KT > 0) {
+#pragma unroll
+    for (int j = 0; j < KT; ++j) tap[j] = ldu<V>(taps + (long)j * H + c);
+  }
+  const int first = blockIdx.x * kConvRows, t1 = min(T, first + kConvRows);
+  int slot_before = -1;
+  for (int t = first; t < t1; ++t) {
+    const int slot = tok_seq[t], pos = tok_pos[t];
+    const Unit<V> h = row_h(t);
+    Unit<V> g = h, s;
+#pragma unroll
+    for (int e = 0; e < V; ++e) s.v[e] = 0.f;
+    if constexpr (KT > 0) {
+      if (t > first && slot == slot_before) {
+#pragma unroll
+        for (int j = 0; j + 1 < KT; ++j) win[j] = win[j + 1];
+      } else {
+#pragma unroll
+        for (int j = 0; j + 1 < KT; ++j) win[j] = earlier(t, KT - 1 - j, slot, pos);
+      }
+      win[KT - 1] = h;
+      slot_before = slot;
+#pragma unroll
+      for (int j = 0; j + 1 < KT; ++j)
+#pragma unroll
+        for (int e = 0; e < V; ++e) s.v[e] += tap[j].v[e] * win[j].v[e];
+#pragma unroll
+      for (int e = 0; e < V; ++e) g.v[e] = h.v[e] + (s.v[e] + tap[KT - 1].v[e] * h.v[e]);
+    } else if (taps) {
       for (int j = 0; j < K - 1; ++j) {
-        const int back = K - 1 - j, p = pos - back;
-        if (p < 0) continue;
-        Unit<V> a;
-        if (t - back >= 0 && tok_seq[t - back] == slot && tok_pos[t - back] == p) {
-          a = ldu<V>(x + (long)(t - back) * H + c);
-          const float fb = rs[t - back];
-#pragma unroll
-          for (int e = 0; e < V; ++e) a.v[e] = a.v[e] * fb * w.v[e];
-        } else if (slot >= 0 && slot < state_rows) {
-          a = ldu<V>(carry + ((long)slot * (K - 1) + p % (K - 1)) * H + c);
-        } else {
-          continue;
-        }
-        const Unit<V> q = ldu<V>(taps + (long)j * H + c);
+        const Unit<V> a = earlier(t, K - 1 - j, slot, pos), q = ldu<V>(taps + (long)j * H + c);
 #pragma unroll
         for (int e = 0; e < V; ++e) s.v[e] += q.v[e] * a.v[e];
       }
@@ -258,11 +290,16 @@ extern "C" void dlia_canon_conv(void* out, int out_f32, long ldo, const float* x
   const bool vec = H % 4 == 0 && al16(x) && al16(nw) && al16(taps) && al16(carry) && al16(out) && ldo % 4 == 0;
   const int per = kCanonThreads * (vec ? 4 : 1);
   const dim3 grid((T + kConvRows - 1) / kConvRows, (H + per - 1) / per);
-#define DLIA_CONV(OT, V)                                                                                                        \
-  hipLaunchKernelGGL((canon_conv_kernel<OT, V>), grid, dim3(kCanonThreads), 0, stream, (OT*)out, ldo, x, rs, nw, taps, carry, K, tok_pos, \
-                     tok_seq, T, state_rows, H)
-  if (out_f32) { if (vec) DLIA_CONV(float, 4); else DLIA_CONV(float, 1); }
-  else { if (vec) DLIA_CONV(bf16, 4); else DLIA_CONV(bf16, 1); }
+#define DLIA_CONV(OT, V, KT)                                                                                                        \
+  hipLaunchKernelGGL((canon_conv_kernel<OT, V, KT>), grid, dim3(kCanonThreads), 0, stream, (OT*)out, ldo, x, rs, nw, taps, carry, K, \
+                     tok_pos, tok_seq, T, state_rows, H)
+#define DLIA_CONV_K(OT)                                                                                       \
+  do {                                                                                                        \
+    if (!vec) DLIA_CONV(OT, 1, 0); else if (taps && K == 2) DLIA_CONV(OT, 4, 2); else if (taps && K == 3) DLIA_CONV(OT, 4, 3); \
+    else if (taps && K == 4) DLIA_CONV(OT, 4, 4); else DLIA_CONV(OT, 4, 0);                                   \
+  } while (0)
+  if (out_f32) DLIA_CONV_K(float); else DLIA_CONV_K(bf16);
+#undef DLIA_CONV_K
 #undef DLIA_CONV
 }
 

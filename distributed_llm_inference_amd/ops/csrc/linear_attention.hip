@@ -18,7 +18,8 @@
 // quarter of 16 tokens keeps its own references: q carries exp(G_i - G_start of i's quarter), k carries exp(G_end of j's quarter -
 // G_j), both at most one, and the score tile of two quarters gets the factor between the two references, which is at most one for
 // different quarters. Inside a quarter that factor is exp(-(the quarter's sum)): where it grows large (a sum below
-// -40), the tile's pairs are summed one by one from exp(G_i - G_j) itself.
+// -60 in log2), the tile's pairs are summed one by one from exp(G_i - G_j) itself.
+// Log decays are kept in units of log2, so that every factor is one hardware exp2.
 // A portion may start and end anywhere: chunks are counted from the portion's first token, and the split only changes rounding.
 #include "units.h"
 #include "launch.h"
@@ -29,7 +30,8 @@ constexpr int kLaChunk = 64;
 constexpr int kLaQuarter = 16;
 constexpr int kLaCh = 64;              // key channels at a time
 constexpr int kLaVals = 128;           // value columns at a time in `local`
-constexpr float kLaFar = -40.f;
+constexpr float kLaFar = -60.f;        // (in log2)
+constexpr float kLaLog2e = 1.4426950408889634f;
 
 struct LaArgs {
   void* out; long ldo;
@@ -43,12 +45,14 @@ struct LaArgs {
   int H, d, dv, rank, state_rows, nblk;
   int col_q, col_k, col_v, col_g, col_a;
   float qscale, inv_tau, eps;
+  int vec;                             // value columns of z come in aligned groups of four
 };
 
 // base^n for log2(base) = l2 (minus infinity for base 0)
 __device__ __forceinline__ float pow_n(int n, float l2) { return n == 0 ? 1.f : exp2f((float)n * l2); }
 __device__ __forceinline__ float log_sigmoid(float x) { return fminf(x, 0.f) - log1pf(expf(-fabsf(x))); }
 __device__ __forceinline__ float la_gate(float g) { return g / (1.f + expf(-g)); }
+__device__ __forceinline__ float ex2(float x) { return __builtin_amdgcn_exp2f(x); }
 __device__ __forceinline__ f32x4 mfma4(float a, float b, f32x4 c) { return __builtin_amdgcn_mfma_f32_16x16x4f32(a, b, c, 0, 0, 0); }
 
 // ---- single tokens --------------------------------------------------------------------------------------------------
@@ -156,16 +160,31 @@ __global__ __launch_bounds__(256) void la_local_kernel(LaArgs p) {
     const float bias = p.a_b[ac];
 #pragma unroll
     for (int i = 0; i < kLaQuarter; ++i) f[i] = bias;
-    for (int r = 0; r < p.rank; ++r) {
-      const float w = p.a2t[(long)r * p.H * d + ac];
-#pragma unroll
-      for (int i = 0; i < kLaQuarter; ++i) f[i] += zq[(long)min(qt * kLaQuarter + i, nt - 1) * p.ldz + p.col_a + r] * w;
+    // the chunk's low-rank projections go through LDS (the values' buffer, not in use yet)
+    const bool staged = p.rank <= VST;
+    if (staged) {
+      for (int i = tid; i < nt * p.rank; i += 256) vs[i] = zq[(long)(i / p.rank) * p.ldz + p.col_a + i % p.rank];
+      __syncthreads();
     }
+    const float* low = staged ? vs : zq + p.col_a;
+    const long lrow = staged ? p.rank : p.ldz;
+    for (int r0 = 0; r0 < p.rank; r0 += 4) {
+      float w[4];
+#pragma unroll
+      for (int u = 0; u < 4; ++u) w[u] = r0 + u < p.rank ? p.a2t[(long)(r0 + u) * p.H * d + ac] : 0.f;
+#pragma unroll
+      for (int u = 0; u < 4; ++u)
+        if (r0 + u < p.rank) {
+#pragma unroll
+          for (int i = 0; i < kLaQuarter; ++i) f[i] += low[min(qt * kLaQuarter + i, nt - 1) * lrow + r0 + u] * w[u];
+        }
+    }
+    const float unit = p.inv_tau * kLaLog2e;
     float run = 0.f;
 #pragma unroll
     for (int i = 0; i < kLaQuarter; ++i) {
       const int row = qt * kLaQuarter + i;
-      if (row < nt) run += log_sigmoid(f[i]) * p.inv_tau;
+      if (row < nt) run += log_sigmoid(f[i]) * unit;
       f[i] = run;
       if (ok && row < nt) p.g[(tq + row) * p.H * d + ac] = run;
     }
@@ -173,9 +192,9 @@ __global__ __launch_bounds__(256) void la_local_kernel(LaArgs p) {
     __syncthreads();
     float rest = run;
     for (int j = qt + 1; j < 4; ++j) rest += tot[j][c];
-    if (qt == 0 && ok) p.ws_dec[crow * p.H * d + ac] = expf(rest);
+    if (qt == 0 && ok) p.ws_dec[crow * p.H * d + ac] = ex2(rest);
 #pragma unroll
-    for (int i = 0; i < kLaQuarter; ++i) f[i] = qt * kLaQuarter + i < nt ? expf(rest - f[i]) : 0.f;
+    for (int i = 0; i < kLaQuarter; ++i) f[i] = qt * kLaQuarter + i < nt ? ex2(rest - f[i]) : 0.f;
   }
 #pragma unroll
   for (int i = 0; i < kLaQuarter; ++i) {
@@ -186,9 +205,26 @@ __global__ __launch_bounds__(256) void la_local_kernel(LaArgs p) {
   float* dst = p.ws_state + (crow * p.H + h) * (long)d * dv;
   for (int v0 = 0; v0 < dv; v0 += kLaVals) {
     __syncthreads();
-    for (int i = tid; i < kLaChunk * kLaVals; i += 256) {
-      const int row = i / kLaVals, cc = i % kLaVals;
-      vs[row * VST + cc] = row < nt && v0 + cc < dv ? zq[(long)row * p.ldz + p.col_v + (long)h * dv + v0 + cc] : 0.f;
+    {
+      // every thread: four neighbouring columns of every eighth token, all loads in flight before the first is parked
+      const int cc = (tid & 31) * 4, r8 = tid >> 5;
+      const float* src = zq + p.col_v + (long)h * dv + v0 + cc;
+      f32x4 v[kLaChunk / 8];
+#pragma unroll
+      for (int i = 0; i < kLaChunk / 8; ++i) {
+        const int row = r8 + i * 8;
+        v[i] = f32x4{0.f, 0.f, 0.f, 0.f};
+        if (row < nt) {
+          if (p.vec) { if (v0 + cc < dv) v[i] = *reinterpret_cast<const f32x4*>(src + (long)row * p.ldz); }
+          else {
+#pragma unroll
+            for (int e = 0; e < 4; ++e)
+              if (v0 + cc + e < dv) v[i][e] = src[(long)row * p.ldz + e];
+          }
+        }
+      }
+#pragma unroll
+      for (int i = 0; i < kLaChunk / 8; ++i) *reinterpret_cast<f32x4*>(vs + (r8 + i * 8) * VST + cc) = v[i];
     }
     __syncthreads();
     if (db * kLaCh + wave * 16 >= d) continue;               // (no barrier until the next round's, which every wave reaches)
@@ -312,8 +348,8 @@ __global__ __launch_bounds__(512) void la_out_kernel(LaArgs p) {
           k = zq[(long)row * p.ldz + p.col_k + h * d + ch];
           if constexpr (!HEAD) {
             const float g = p.g[(tq + row) * p.H * d + gc];
-            q *= expf(g);
-            k *= expf(total - g);
+            q *= ex2(g);
+            k *= ex2(total - g);
           }
         }
         qs[row * ST + c] = q;
@@ -339,7 +375,7 @@ __global__ __launch_bounds__(512) void la_out_kernel(LaArgs p) {
             for (int r = 0; r < 4; ++r) {
               const int i = I * 16 + kq * 4 + r;
               if (i >= j && i < nt)
-                sc[s][r] += zq[(long)i * p.ldz + p.col_q + h * d + ch] * p.qscale * k * expf(p.g[(tq + i) * p.H * d + (long)h * d + ch] - gj);
+                sc[s][r] += zq[(long)i * p.ldz + p.col_q + h * d + ch] * p.qscale * k * ex2(p.g[(tq + i) * p.H * d + (long)h * d + ch] - gj);
             }
           }
           continue;
@@ -355,7 +391,7 @@ __global__ __launch_bounds__(512) void la_out_kernel(LaArgs p) {
           for (int e = 0; e < 4; ++e) {
             float f = I == J ? -tot[I][c + e] : 0.f;
             for (int m = J + 1; m < I; ++m) f += tot[m][c + e];
-            qa[e] *= expf(f);
+            qa[e] *= ex2(f);
           }
         }
 #pragma unroll
@@ -375,7 +411,7 @@ __global__ __launch_bounds__(512) void la_out_kernel(LaArgs p) {
             float f = 0.f;
 #pragma unroll
             for (int m = 0; m < I; ++m) f += tot[m][c + e];
-            if (I > 0) qa[e] *= expf(f);
+            if (I > 0) qa[e] *= ex2(f);
           }
         }
 #pragma unroll
@@ -486,8 +522,9 @@ extern "C" int dlia_linear_attention(void* out, int out_f32, long ldo, const flo
   p.nblk = (d + kLaCh - 1) / kLaCh;
   p.ws_state = p.ws_dec = p.g = nullptr;
   const bool vec = dv % 4 == 0 && (uintptr_t)state % 16 == 0;
+  p.vec = dv % 4 == 0 && col_v % 4 == 0 && ldz % 4 == 0 && (uintptr_t)z % 16 == 0;
   if (max_q == 1) {
-    const bool v4 = vec && col_v % 4 == 0 && ldz % 4 == 0 && (uintptr_t)z % 16 == 0;
+    const bool v4 = vec && p.vec;
     const int units = v4 ? dv / 4 : dv, CT = units < 256 ? units : 256;
     const size_t lds = ((3 * d + 3) / 4 * 4 + (256 / CT) * dv) * sizeof(float);
     const dim3 grid(H, B);

@@ -587,19 +587,20 @@ __global__ __launch_bounds__(256) void tile_merge_kernel(bf16* __restrict__ out,
 #pragma unroll
   for (int a = 0; a < MAPS; ++a) {
     const float* pr = part + (((long)t * H + h) * MAPS + a) * nz * (dv + 2);
-    float M = -INFINITY;
-    for (int z = 0; z < nz; ++z) M = fmaxf(M, pr[(long)z * (dv + 2) + dv]);
-    float L = 0.f;
+    // lane z holds split z's maximum and sum (up to 16 splits); the splits' weights then travel by lane broadcast, so that the loads
+    // of all splits' values are independent of each other (a split that saw no key has weight 0)
+    const float mz = lane < nz ? pr[(long)lane * (dv + 2) + dv] : -INFINITY;
+    const float M = wave_max(mz);
+    const float wz = mz == -INFINITY ? 0.f : expf(mz - M);
+    float L = wave_sum(wz > 0.f ? wz * pr[(long)lane * (dv + 2) + dv + 1] : 0.f);
 #pragma unroll
     for (int c = 0; c < kMultiMaxDV / 64; ++c) o[a][c] = 0.f;
+#pragma unroll 4
     for (int z = 0; z < nz; ++z) {
       const float* pz = pr + (long)z * (dv + 2);
-      const float mz = pz[dv];
-      if (mz == -INFINITY) continue;                  // (uniform: a split that saw no key)
-      const float w = expf(mz - M);
-      L += pz[dv + 1] * w;
+      const float w = __shfl(wz, z, 64);
 #pragma unroll
-      for (int c = 0; c < kMultiMaxDV / 64; ++c) { const int col = c * 64 + lane; if (col < dv) o[a][c] += pz[col] * w; }
+      for (int c = 0; c < kMultiMaxDV / 64; ++c) { const int col = c * 64 + lane; if (col < dv) { const float v = pz[col] * w; o[a][c] += w > 0.f ? v : 0.f; } }
     }
     if (sink) L = M == -INFINITY ? 1.f : L + expf(sink[h] - M);
     const float inv = L > 0.f ? 1.f / L : 0.f;
