@@ -757,7 +757,10 @@ class GpuStage:
             if st.graph is None or st.splits != st.splits_wanted:
                 st.splits = st.splits_wanted
                 self._capture(st)
-            st.graph.replay()
+            # (torch refuses to start a replay while the calling thread's stream reports a capture, which the default stream does
+            # when another stage thread of this process is in one: wait for it)
+            with _CAPTURE_LOCK:
+                st.graph.replay()
             self.graph_replays += 1
         return st.tokens if self.plan.has_head else st.hidden_out
 
