@@ -99,10 +99,15 @@ class LayerSpec:
     ``latent_attention`` without a query latent (`q_rank` 0) projects its queries from the mixer's input directly; `window`
     limits it as above; `kv_from` = j >= 0: the layer keeps nothing of its own and reads layer j's latents and rotated key
     parts (its own query, key and value projections, window and scale).
+    Further switches of ``attention``: `head_norm`: every head's q and k are RMS-normed over their `dim` entries ahead of the
+    rotation, with one learned weight for all query heads and one for all key heads. `unit_qk`: every head's q and k are divided
+    by their root mean square AFTER the rotation (no weight). `k_values`: there is no value projection, the values are the keys
+    as projected (ahead of norm and rotation).
     The feed-forward sublayer is `ff_kind`: ``gated_gelu`` (gelu_tanh(gate) * up, biases), ``gelu`` (up, exact
     GELU, down; no biases), ``xielu`` (up, a two-sided quadratic / exponential unit with two learned numbers, down),
     ``relu2`` (up, the square of relu, down; biases), ``polynorm`` (up, a N(z) + b N(z^2) + c N(z^3) + e with four learned
-    numbers, N dividing a token's row by its root mean square, down) or ``moe`` (`moe` says how tokens are routed to its experts)."""
+    numbers, N dividing a token's row by its root mean square, down), ``relu_glu`` (relu(gate) * up, down; no biases) or ``moe``
+    (`moe` says how tokens are routed to its experts)."""
     # "attention" | "delta" | "general_delta" | "mlstm" | "parallel" | "rglru" | "latent_attention" | "linear_attention"
     kind: str
     heads: int
@@ -150,6 +155,9 @@ class LayerSpec:
     tau: float = 1.0
     o_norm: bool = False
     kv_from: int = -1
+    head_norm: bool = False
+    unit_qk: bool = False
+    k_values: bool = False
 
     @property
     def group(self) -> int:
@@ -198,14 +206,19 @@ class LayerSpec:
         if self.kind == "mlstm":
             return width * self.heads * (2 * self.dim + 3 * self.vdim + 2) + 2 * self.heads + self.heads * self.vdim
         qn, kn, vn = self.qk_heads * self.dim, self.kv_heads * self.dim, self.v_heads * self.vdim
-        n = width * (qn + kn + vn) + self.heads * self.vdim * width
+        n = width * (qn + kn + (0 if self.k_values else vn)) + (2 if self.out_gate else 1) * self.heads * self.vdim * width
+        if self.kind == "attention" and (self.head_norm or self.unit_qk):
+            return n + (2 * self.dim if self.head_norm else 0)
         if self.kind == "attention":
             return n + qn + kn + vn + 1
         return n + self.conv * (qn + kn + vn) + 2 * self.heads * width + 2 * self.heads + self.vdim + self.heads * self.vdim * width
 
     def ff_param_count(self, width: int) -> int:
         if self.moe is not None:
-            return self.moe.experts * (3 * width * self.moe.ff + width) + 3 * width * self.moe.shared_ff
+            mats = 2 if self.moe.act == "relu2" else 3
+            return self.moe.experts * (mats * width * self.moe.ff + width) + mats * width * self.moe.shared_ff
+        if self.ff_kind == "relu_glu":
+            return 3 * width * self.ff
         if self.ff_kind in ("gelu", "xielu", "polynorm"):
             return 2 * width * self.ff
         if self.ff_kind == "relu2":
@@ -229,7 +242,9 @@ class MoeSpec:
     the groups. `shared_ff` > 0: one more expert of that width runs for every token and is added unweighted, or (`shared_gate`)
     multiplied by the sigmoid of one more projection of the token to a single number; `shared_limit` is its activation's limit.
     `act` ``silu``: an expert computes down(silu(gate(x)) * up(x)), no limits. `score` ``table``: there is no router; a table
-    [vocab, top] of expert numbers names each token's experts by the token's id, each weighted 1 / top."""
+    [vocab, top] of expert numbers names each token's experts by the token's id, each weighted 1 / top. `act` ``relu2``: an
+    expert computes down(relu(up(x))^2), there is no gate. `input_weight`: the weight multiplies what the expert READS, the
+    experts' outputs are added as they are."""
     experts: int
     top: int
     ff: int
@@ -246,6 +261,7 @@ class MoeSpec:
     act: str = "swish_lim"
     shared_gate: bool = False
     shared_limit: float = 0.0
+    input_weight: bool = False
 
     @property
     def outputs(self) -> int:
@@ -256,7 +272,7 @@ class MoeSpec:
 @dataclass(frozen=True)
 class ModelSpec:
     name: str
-    family: str                     # "llama" | "gpt2" | "letarax" | "nufapel" | "tezesun" | "zovozen" | "pifutar"
+    family: str                     # "llama" | "gpt2" | "letarax" | "nufapel" | "tezesun" | "zovozen" | "pifutar" | "migenex"
     num_layers: int
     hidden_size: int
     num_heads: int
@@ -290,7 +306,7 @@ class ModelSpec:
     norm_kind: str = "rms"
     gated_residual: bool = False
     # (start, stop, times): layers start .. stop-1 run `times` times in a row with the same weights, every pass with a
-    # cache / state of its own and behind a learned vector added to the residual stream
+    # cache / state of its own and behind a learned vector added to the residual stream (or, with `loop_input`, behind a linear map)
     loop: tuple = ()
     learned_positions: bool = False          # a learned vector per position is added to the embedding
     logit_softcap: float = 0.0               # > 0: logits <- cap tanh(logits / cap)
@@ -309,6 +325,16 @@ class ModelSpec:
     # what goes on from a layer is a learned weighted sum of the embedding and of all layers' results so far
     input_conv: int = 0
     depth_average: bool = False
+    # `sandwich`: plain-weight RMS norms before and after every sublayer, the normed output times `residual_mult`:
+    # x += residual_mult * norm1b(mixer(norm1(x))), the same for the feed-forward. `loop_input`: a pass of the repeated stretch
+    # starts from x <- W [x; x0], x0 the embedding output (also the first pass)
+    sandwich: bool = False
+    residual_mult: float = 1.0
+    loop_input: bool = False
+    # the embedding rows are multiplied by `embed_scale`; `bigram` (buckets, mul_prev, mul_cur): row (previous token * mul_prev +
+    # token * mul_cur) mod buckets of a second table is added, row `buckets` for a sequence's first token
+    embed_scale: float = 1.0
+    bigram: tuple = ()
 
     @property
     def is_hybrid(self) -> bool:
@@ -682,6 +708,96 @@ class ModelSpec:
             bos_token_id=cfg.get("bos_token_id"), eos_token_id=_scalar_eos(cfg.get("eos_token_id")), hf_type="pifutar",
             layer_specs=tuple(layers), input_conv=int((cfg.get("canon") or {}).get("taps") or 0), depth_average=True)
 
+    @staticmethod
+    def from_migenex_config(cfg: Dict[str, Any], name: str = "") -> "ModelSpec":
+        """Migenex: sandwich-norm layers with a residual multiplier. ``layers`` lists for each layer its ``type`` —
+        ``attention`` (mixer: heads, kv_heads, dim, vdim, scale, softcap, rot.dims / base: normed heads, halves rotated, the whole
+        context) or ``attention_2`` (heads, kv_heads, dim, vdim, scale, mask.size = window, rot.dims / base: the keys are the
+        values, pairs rotated, unit heads, output gate) — and its ``mlp``: null, ``dense`` (ff) or ``moe`` (expert.ff,
+        router.experts / top, shared.ff). ``embedding``: scale and bigram (buckets, mul_prev, mul_cur); ``loop`` (start, stop,
+        times) repeats a stretch of layers, each pass behind a map of the stream and the embedding output. A head of its own.
+        Keys a config leaves out switch their mechanism off."""
+        layers = []
+        for i, l in enumerate(cfg["layers"]):
+            m, mlp = l["mixer"], l.get("mlp")
+            ffkw: Dict[str, Any] = dict(ff=0, ff_kind="relu_glu")
+            if mlp is not None and mlp.get("kind", "dense") == "dense":
+                ffkw = dict(ff=int(mlp["ff"]), ff_kind="relu_glu")
+            elif mlp is not None and mlp["kind"] == "moe":
+                r = mlp["router"]
+                moe = MoeSpec(experts=int(r["experts"]), top=int(r["top"]), ff=int(mlp["expert"]["ff"]), limit=0.0, group_rank=1, renorm=False,
+                              shared_ff=int((mlp.get("shared") or {}).get("ff") or 0), act="relu2", input_weight=True)
+                if not 1 <= moe.top <= moe.experts:
+                    raise ValueError(f"layer {i}: {moe.experts} experts, {moe.top} chosen")
+                ffkw = dict(ff=0, ff_kind="moe", moe=moe)
+            elif mlp is not None:
+                raise ValueError(f"layer {i}: feed-forward kind {mlp.get('kind')!r} is not supported (dense and moe are)")
+            H, G, d, dv = (int(m[k]) for k in ("heads", "kv_heads", "dim", "vdim"))
+            if H % G:
+                raise ValueError(f"layer {i}: {H} heads over {G} key / value heads")
+            rot = m.get("rot") or {}
+            rd = int(rot.get("dims") or 0)
+            if rd % 2 or rd > d:
+                raise ValueError(f"layer {i}: {rd} rotated entries of {d}")
+            win = (m.get("mask") or {}).get("size")
+            common = dict(heads=H, kv_heads=G, dim=d, vdim=dv, scale=float(m.get("scale", d ** -0.5)), window=int(win) if win else None,
+                          softcap=float(m.get("softcap") or 0.0), rope_dims=rd, rope_base=float(rot.get("base", 10000.0)), **ffkw)
+            if l["type"] == "attention":
+                layers.append(LayerSpec("attention", head_norm=True, **common))
+            elif l["type"] == "attention_2":
+                if dv != d:
+                    raise ValueError(f"layer {i}: values of {dv} entries cannot be the keys of {d}")
+                layers.append(LayerSpec("attention", unit_qk=True, k_values=True, out_gate=True, rope_interleaved=True, **common))
+            else:
+                raise ValueError(f"layer {i}: unknown mixer type {l['type']!r}")
+        if not layers:
+            raise ValueError("a model needs at least one layer")
+        lp, loop = (), cfg.get("loop") or None
+        if loop:
+            lp = (int(loop["start"]), int(loop["stop"]), int(loop["times"]))
+            if not 0 <= lp[0] < lp[1] <= len(layers) or lp[2] < 1:
+                raise ValueError(f"loop {lp} does not fit {len(layers)} layers")
+        emb = cfg.get("embedding") or {}
+        big = emb.get("bigram") or None
+        return ModelSpec(
+            name=name or "migenex", family="migenex", num_layers=len(layers), hidden_size=int(cfg["width"]),
+            num_heads=max(l.heads for l in layers), num_kv_heads=max(l.kv_heads for l in layers),
+            head_dim=max(max(l.dim, l.vdim) for l in layers),
+            intermediate_size=max(max(l.ff, l.moe.ff if l.moe else 0, l.moe.shared_ff if l.moe else 0) for l in layers),
+            vocab_size=int(cfg["vocab"]), max_position=1 << 30, norm_eps=float(cfg["norm"]["eps"]), tie_embeddings=False,
+            bos_token_id=cfg.get("bos_token_id"), eos_token_id=_scalar_eos(cfg.get("eos_token_id")), hf_type="migenex",
+            layer_specs=tuple(layers), loop=lp, sandwich=True, residual_mult=float(cfg.get("residual_mult", 1.0)), loop_input=bool(lp),
+            embed_scale=float(emb.get("scale", 1.0)),
+            bigram=(int(big["buckets"]), int(big["mul_prev"]), int(big["mul_cur"])) if big else ())
+
+    def migenex_config(self) -> Dict[str, Any]:
+        """The inverse of `from_migenex_config`."""
+        out = []
+        for l in self.layer_specs:
+            m: Dict[str, Any] = {"heads": l.heads, "kv_heads": l.kv_heads, "dim": l.dim, "vdim": l.vdim, "scale": l.scale}
+            if l.rope_dims:
+                m["rot"] = {"base": l.rope_base, "dims": l.rope_dims}
+            if l.window:
+                m["mask"] = {"size": l.window}
+            if l.softcap > 0:
+                m["softcap"] = l.softcap
+            if l.moe is not None:
+                e = l.moe
+                mlp: Optional[Dict[str, Any]] = {"kind": "moe", "expert": {"ff": e.ff}, "router": {"experts": e.experts, "top": e.top}}
+                if e.shared_ff:
+                    mlp["shared"] = {"ff": e.shared_ff}
+            else:
+                mlp = {"kind": "dense", "ff": l.ff} if l.ff else None
+            out.append({"type": "attention_2" if l.k_values else "attention", "mixer": m, "mlp": mlp})
+        emb: Dict[str, Any] = {"scale": self.embed_scale}
+        if self.bigram:
+            emb["bigram"] = dict(zip(("buckets", "mul_prev", "mul_cur"), self.bigram))
+        cfg = {"architecture": "Migenex", "embedding": emb, "layers": out, "norm": {"eps": self.norm_eps}, "residual_mult": self.residual_mult,
+               "vocab": self.vocab_size, "width": self.hidden_size, "bos_token_id": self.bos_token_id, "eos_token_id": self.eos_token_id}
+        if self.loop:
+            cfg["loop"] = dict(zip(("start", "stop", "times"), self.loop))
+        return cfg
+
     def pifutar_config(self) -> Dict[str, Any]:
         """The inverse of `from_pifutar_config` (`rank` is a size a checkpoint's tensors give; it is written so that random
         weights of the same shapes can be drawn from the config alone)."""
@@ -825,6 +941,8 @@ class ModelSpec:
             return ModelSpec.from_zovozen_config(cfg, name=name)
         if cfg.get("architecture") == "Pifutar":
             return ModelSpec.from_pifutar_config(cfg, name=name)
+        if cfg.get("architecture") == "Migenex":
+            return ModelSpec.from_migenex_config(cfg, name=name)
         if mt == "gpt2" or any("GPT2" in a for a in archs):
             if cfg.get("activation_function", "gelu_new") != "gelu_new" or cfg.get("scale_attn_by_inverse_layer_idx"):
                 raise ValueError("GPT-2 variants other than gelu_new MLPs with plain 1/sqrt(d) attention scaling are not supported")
@@ -957,7 +1075,7 @@ class ModelSpec:
         """The inverse of `from_hf_config`: a config.json dict for this spec."""
         if self.is_hybrid:
             return {"nufapel": self.nufapel_config, "tezesun": self.tezesun_config, "zovozen": self.zovozen_config,
-                    "pifutar": self.pifutar_config}.get(self.family, self.letarax_config)()
+                    "pifutar": self.pifutar_config, "migenex": self.migenex_config}.get(self.family, self.letarax_config)()
         if self.is_gpt2:
             return {
                 "model_type": "gpt2", "architectures": ["GPT2LMHeadModel"],
@@ -1186,6 +1304,34 @@ def pifutar_spec(name: str, width: int, heads: int, head_dim: int, ff: int, num_
                      eos_token_id=2, hf_type="pifutar", layer_specs=tuple(layers), input_conv=taps, depth_average=True)
 
 
+def migenex_spec(name: str, width: int, heads: int, kv_heads: int, head_dim: int, ff: int, num_layers: int, window: int, vocab_size: int = 32000,
+                 pattern: str = "wwwf", dense: str = "dm", experts: int = 8, top: int = 1, loop: tuple = (), full_heads: int = 0, full_kv: int = 0,
+                 full_dim: int = 0, full_vdim: int = 0, rot_dims: int = 0, buckets: int = 65521, residual_mult: float = 0.4) -> ModelSpec:
+    """A Migenex stack from a few numbers: `pattern` repeats over the layers ('w' windowed attention over its own keys as values,
+    unit heads, pairs rotated, output gate; 'f' attention over the whole context, normed heads, halves rotated, capped scores);
+    `dense` repeats over the layers' feed-forwards: 'd' dense of `ff`, 'm' routed (`experts` experts of ff / 4, `top` per token,
+    a shared expert of ff / 2), 'n' none."""
+    moe = MoeSpec(experts=experts, top=top, ff=max(8, ff // 4), limit=0.0, group_rank=1, renorm=False, shared_ff=max(8, ff // 2), act="relu2",
+                  input_weight=True)
+    fd = full_dim or head_dim
+    layers = []
+    for i in range(num_layers):
+        f = dense[i % len(dense)]
+        kw: Dict[str, Any] = dict(ff=ff, ff_kind="relu_glu") if f == "d" else dict(ff=0, ff_kind="relu_glu") if f == "n" else dict(ff=0, ff_kind="moe", moe=moe)
+        if pattern[i % len(pattern)] == "w":
+            layers.append(LayerSpec("attention", heads=heads, kv_heads=kv_heads, dim=head_dim, vdim=head_dim, window=window, scale=head_dim ** -0.5,
+                                    unit_qk=True, k_values=True, out_gate=True, rope_dims=rot_dims or head_dim, rope_base=10000.0,
+                                    rope_interleaved=True, **kw))
+        else:
+            layers.append(LayerSpec("attention", heads=full_heads or heads, kv_heads=full_kv or kv_heads, dim=fd, vdim=full_vdim or fd,
+                                    scale=fd ** -0.5, softcap=50.0, head_norm=True, rope_dims=min(rot_dims or fd, fd), rope_base=500000.0, **kw))
+    return ModelSpec(name=name, family="migenex", num_layers=num_layers, hidden_size=width, num_heads=max(l.heads for l in layers),
+                     num_kv_heads=max(l.kv_heads for l in layers), head_dim=max(max(l.dim, l.vdim) for l in layers), intermediate_size=ff,
+                     vocab_size=vocab_size, max_position=1 << 30, norm_eps=1e-5, tie_embeddings=False, bos_token_id=1, eos_token_id=2,
+                     hf_type="migenex", layer_specs=tuple(layers), loop=loop, sandwich=True, residual_mult=residual_mult, loop_input=bool(loop),
+                     embed_scale=float(width) ** 0.5, bigram=(buckets, 31337, 7919) if buckets else ())
+
+
 # Letarax stacks of the sizes of the Llama benchmark shapes (random weights; `bench.py --hybrid-compare` runs them)
 BUILTIN_SPECS["letarax-1b-like"] = letarax_spec("letarax-1b-like", 2048, 16, 4, 128, 8192, 8, 1024)
 BUILTIN_SPECS["letarax-8b-like"] = letarax_spec("letarax-8b-like", 4096, 32, 8, 128, 14336, 4, 2048)
@@ -1201,6 +1347,9 @@ BUILTIN_SPECS["zovozen-8b-like"] = zovozen_spec("zovozen-8b-like", 4096, 32, 8, 
 # Pifutar stacks of the same sizes (`bench.py --canon-compare` runs them beside the Tezesun and Nufapel stacks)
 BUILTIN_SPECS["pifutar-1b-like"] = pifutar_spec("pifutar-1b-like", 2048, 16, 128, 8192, 8, window=1024, kv_rank=448, rot_dim=64)
 BUILTIN_SPECS["pifutar-8b-like"] = pifutar_spec("pifutar-8b-like", 4096, 32, 128, 14336, 4, window=2048, kv_rank=448, rot_dim=64)
+# Migenex stacks of the same sizes (`bench.py --sandwich-compare` runs them beside the Letarax and Nufapel stacks)
+BUILTIN_SPECS["migenex-1b-like"] = migenex_spec("migenex-1b-like", 2048, 16, 4, 128, 8192, 8, window=1024, loop=(0, 4, 1))
+BUILTIN_SPECS["migenex-8b-like"] = migenex_spec("migenex-8b-like", 4096, 32, 8, 128, 14336, 4, window=2048, loop=(0, 4, 1))
 
 
 def _register_test_models():
@@ -1232,6 +1381,12 @@ def _register_test_models():
                                                       kv_rank=20, rot_dim=8, vdim=24, rank=4, taps=3, dense="-d-n-")
     BUILTIN_SPECS["tiny-pifutar-gpu-test"] = pifutar_spec("tiny-pifutar-gpu-test", 128, 4, 32, 256, 5, window=36, vocab_size=320, pattern="rglsg",
                                                           experts=6, kv_rank=40, rot_dim=16, vdim=48, rank=8, taps=4, dense="d--")
+    BUILTIN_SPECS["tiny-migenex-test"] = migenex_spec("tiny-migenex-test", 64, 4, 2, 16, 96, 5, window=13, vocab_size=320, pattern="wfw", dense="mdnm",
+                                                      experts=5, top=2, loop=(1, 3, 2), full_heads=6, full_kv=3, full_dim=20, full_vdim=12,
+                                                      rot_dims=12, buckets=101)
+    BUILTIN_SPECS["tiny-migenex-gpu-test"] = migenex_spec("tiny-migenex-gpu-test", 128, 4, 2, 64, 256, 5, window=37, vocab_size=320, pattern="wfw",
+                                                          dense="md", experts=6, top=2, loop=(0, 2, 3), full_dim=32, full_vdim=48, rot_dims=24,
+                                                          buckets=211)
     BUILTIN_SPECS["tiny-gpt2-gpu-test"] = tiny_spec(
         "gpt2", name="tiny-gpt2-gpu-test", hidden_size=256, num_heads=4, num_kv_heads=4, head_dim=64,
         intermediate_size=1024, vocab_size=333, num_layers=4)

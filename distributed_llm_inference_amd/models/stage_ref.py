@@ -54,9 +54,11 @@ class RefStage:
     def _slot_cache(self, slot: int):
         c = self.cache.get(slot)
         if c is None:
-            if self.spec.is_hybrid and self.spec.norm_kind == "dyt":
+            if self.spec.is_hybrid and (self.spec.norm_kind == "dyt" or self.spec.sandwich):
                 # one entry per layer RUN (a repeated stretch of layers owns a cache / state per pass)
                 c = [self._fresh_layer_state(self.spec.layer_specs[i]) for i, _ in self.spec.layer_runs()]
+                if self.spec.bigram:                # and the sequence's tokens
+                    c.append([torch.zeros(0, dtype=torch.long, device=self.device)])
             elif self.spec.is_hybrid:
                 c = [self._fresh_layer_state(self.spec.layer_specs[i]) for i in self.plan.layers]
                 if self.spec.token_shift:           # every layer also carries the previous token's normed input
@@ -539,10 +541,104 @@ class RefStage:
             self.layer_outputs.append(h)
         return h
 
+    # -- hybrid stacks with plain-weight norms on both sides of every sublayer, a residual multiplier and mapped passes ----
+    def _sandwich_embed(self, seqs, ids: torch.Tensor) -> torch.Tensor:
+        """embed[token] * scale, plus the bigram table's row of (previous token, token); the tokens of earlier portions
+        are kept with the sequence."""
+        spec = self.spec
+        x = self.w.embed[ids].float() * spec.embed_scale
+        if spec.bigram:
+            buckets, mp, mc = spec.bigram
+            row = torch.empty_like(ids)
+            for slot, s0, qlen, ctx in seqs:
+                st = self._slot_cache(slot)[-1]
+                cur = ids[s0:s0 + qlen]
+                st[0] = torch.cat([st[0][:ctx], cur])
+                prev = st[0][ctx - 1:-1] if ctx else torch.cat([cur[:1], cur[:-1]])
+                row[s0:s0 + qlen] = (prev * mp + cur * mc) % buckets
+                if ctx == 0:
+                    row[s0] = buckets
+            x = x + self.w.bigram[row].float()
+        return x
+
+    def _sandwich_layers(self, batch: StepBatch, ids: torch.Tensor) -> torch.Tensor:
+        """x <- x + m norm1b(mixer(norm1(x))), x <- x + m norm2b(ff(norm2(x))) for every layer run, x <- W [x; x0] ahead of every
+        pass of the repeated stretch. Attention with normed or unit heads, either rotation, capped scores, a window, keys as values, an
+        output gate; dense relu-gated or routed squared-relu feed-forward (experts on their weighted input, shared expert). Norms,
+        rotations, scores, routers and the residual sum are fp32 whatever the dtype."""
+        from .rope import rope_table
+        spec, dt, eps, w, m = self.spec, self.dtype, self.spec.norm_eps, self.w, self.spec.residual_mult
+        T, dev = ids.numel(), self.device
+        lin = lambda x, mat: R.gemm(x.to(dt), mat, None, None, 0)
+        rnd = lambda x: x.to(dt).float()
+        seqs, t0 = [], 0
+        for slot, qlen, ctx in zip(batch.slots, batch.q_lens, batch.ctx_lens):
+            if qlen > 0 and ctx == 0:
+                self.cache.pop(slot, None)            # a sequence's first tokens: whatever the slot held before is void
+            if qlen > 0:
+                seqs.append((slot, t0, qlen, ctx))
+            t0 += qlen
+        pos = torch.tensor([c + i for c, q in zip(batch.ctx_lens, batch.q_lens) for i in range(q)], dtype=torch.long, device=dev)
+        far = int(pos.max()) + 1 if T else 1
+        x0 = h = self._sandwich_embed(seqs, ids)
+        self.layer_outputs = []
+        for ri, (li, pas) in enumerate(spec.layer_runs()):
+            ls, l = spec.layer_specs[li], w.layers[li]
+            if spec.loop_input and pas >= 0 and li == spec.loop[0]:
+                h = lin(torch.cat([h, x0], dim=1), w.loop_in)
+            H, G, d, dv = ls.heads, ls.kv_heads, ls.dim, ls.vdim
+            z = lin(R.rmsnorm(h, l["ln1_w"], eps), l["w_in"])
+            q, k = z[:, :H * d].reshape(T, H, d), z[:, H * d:(H + G) * d].reshape(T, G, d)
+            v = k if ls.k_values else z[:, (H + G) * d:(H + G) * d + G * dv].reshape(T, G, dv)
+            if ls.head_norm:
+                q, k = R.rmsnorm(q, l["q_norm_w"], eps), R.rmsnorm(k, l["k_norm_w"], eps)
+            if ls.rope_dims:
+                cos, sin = rope_table(ls.rope_dims, ls.rope_base, ls.rope_scaling, far, dev)
+                q, k = R.rope_partial(q, cos, sin, pos, ls.rope_interleaved), R.rope_partial(k, cos, sin, pos, ls.rope_interleaved)
+            if ls.unit_qk:
+                q, k = R.rmsnorm(q, torch.ones(d, device=dev), eps), R.rmsnorm(k, torch.ones(d, device=dev), eps)
+            mixed = torch.empty(T, H, dv, dtype=torch.float32, device=dev)
+            for slot, s0, qlen, ctx in seqs:
+                st, sl = self._slot_cache(slot)[ri], slice(s0, s0 + qlen)
+                assert st[0].shape[0] >= ctx, f"slot {slot}: cache has {st[0].shape[0]} tokens, step says {ctx}"
+                st[0] = torch.cat([st[0][:ctx], k[sl].to(dt)])
+                st[1] = torch.cat([st[1][:ctx], v[sl].to(dt)])
+                mixed[sl] = R.attention(q[sl].to(dt), st[0], st[1], ctx, ls.scale, window=ls.window or 0, softcap=ls.softcap)
+            mixed = mixed.reshape(T, H * dv)
+            if ls.out_gate:
+                mixed = mixed * torch.sigmoid(z[:, -H * dv:])
+            h = h + m * R.rmsnorm(lin(mixed, l["w_o"]), l["ln1b_w"], eps)
+            if ls.has_ff:
+                n = R.rmsnorm(h, l["ln2_w"], eps)
+                if ls.moe is None:
+                    y = lin(rnd(torch.relu(lin(n, l["w_gate"])) * lin(n, l["w_up"])), l["w_down"])
+                else:
+                    e = ls.moe
+                    relu2 = lambda u: torch.relu(u) ** 2
+                    idx, wts = R.moe_route(torch.sigmoid(lin(n, l["w_router"])), e.top, e.groups, e.keep, e.scale, group_rank=e.group_rank, renorm=e.renorm)
+                    y = torch.zeros_like(h)
+                    for ex in range(e.experts):
+                        rows, col = (idx == ex).nonzero(as_tuple=True)
+                        if rows.numel():          # (the weight on the input: up(w n) = w up(n))
+                            y.index_add_(0, rows, lin(rnd(relu2(lin(n[rows], l["w_up_e"][ex]) * wts[rows, col].unsqueeze(1))), l["w_down_e"][ex]))
+                    if e.shared_ff:
+                        y = y + lin(rnd(relu2(lin(n, l["w_up_s"]))), l["w_down_s"])
+                h = h + m * R.rmsnorm(y, l["ln2b_w"], eps)
+            self.layer_outputs.append(h)
+        return h
+
     def _forward_hybrid(self, batch: StepBatch, x: torch.Tensor) -> torch.Tensor:
         T = batch.num_tokens
         ids = torch.as_tensor(x).to(self.device).long().reshape(-1)
         assert ids.numel() == T, f"expected {T} token ids, got {ids.numel()}"
+        if self.spec.sandwich:
+            h = self._sandwich_layers(batch, ids)
+            self.last_hidden = h
+            rows = self._out_rows(batch)
+            if not rows:
+                return torch.empty(0, self.spec.vocab_size, dtype=torch.float32, device=self.device)
+            hn = R.rmsnorm(h[rows], self.w.final_norm_w, self.spec.norm_eps)
+            return R.gemm(hn.to(self.dtype), self.w.lm_head).float()
         if self.spec.input_conv or self.spec.depth_average:
             h = self._canon_layers(batch, self.w.embed[ids].float(), ids)
             self.last_hidden = h

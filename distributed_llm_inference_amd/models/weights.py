@@ -62,6 +62,8 @@ class StageWeights:
     lm_head: Optional[torch.Tensor] = None
     final_norm_a: Optional[torch.Tensor] = None      # dynamic-tanh norms: the scalar inside the tanh
     loop_step: Optional[torch.Tensor] = None         # [passes, H]: added to the residual stream ahead of each pass of a repeated stretch
+    loop_in: Optional[torch.Tensor] = None           # [H, 2 H]: a pass starts from loop_in . [stream; embedding output]
+    bigram: Optional[torch.Tensor] = None            # [buckets + 1, H]: embedding rows by a hash of (previous token, token)
 
     def num_bytes(self) -> int:
         seen, total = set(), 0
@@ -74,7 +76,8 @@ class StageWeights:
         return total
 
     def tensors(self):
-        for t in (self.embed, self.pos_embed, self.final_norm_w, self.final_norm_b, self.lm_head, self.final_norm_a, self.loop_step):
+        for t in (self.embed, self.pos_embed, self.final_norm_w, self.final_norm_b, self.lm_head, self.final_norm_a, self.loop_step,
+                  self.loop_in, self.bigram):
             if t is not None:
                 yield t
         for l in self.layers:
@@ -94,6 +97,7 @@ class StageWeights:
         out.final_norm_w = cv(self.final_norm_w)
         out.final_norm_b = cv(self.final_norm_b)
         out.final_norm_a, out.loop_step = cv(self.final_norm_a), cv(self.loop_step)
+        out.loop_in, out.bigram = cv(self.loop_in), cv(self.bigram)
         out.lm_head = out.embed if tied else cv(self.lm_head)
         return out
 
@@ -608,6 +612,117 @@ def _random_pifutar_weights(spec: ModelSpec, plan: StagePlan, seed: int, device,
     return w
 
 
+# ---- Migenex: checkpoint names <-> the logical layout ---------------------------------------------------------------
+# Per layer: ln1_w, ln1b_w (ln2_w, ln2b_w) the norms before and after a sublayer (plain weights)
+#   mixer: w_in = q | k (| v) (| g) (one GEMM; no v where the keys are the values), w_o, q_norm_w, k_norm_w [dim] with normed heads
+#   dense: w_gate, w_up, w_down      moe: w_router [E, H], w_up_e [E, ff, H], w_down_e [E, H, ff], w_up_s, w_down_s
+def _migenex_layer_names(ls, p: str) -> Dict[str, object]:
+    """logical name -> checkpoint name(s); a tuple is concatenated along the rows, a list stacked."""
+    m, f = p + "mix.", p + "mlp."
+    n: Dict[str, object] = {"ln1_w": p + "norm1", "ln1b_w": p + "norm1b", "w_o": m + "o",
+                            "w_in": tuple(m + x for x in ("q", "k") + (() if ls.k_values else ("v",)) + (("g",) if ls.out_gate else ()))}
+    if ls.head_norm:
+        n["q_norm_w"], n["k_norm_w"] = m + "q.norm", m + "k.norm"
+    if ls.has_ff:
+        n["ln2_w"], n["ln2b_w"] = p + "norm2", p + "norm2b"
+    if ls.moe is not None:
+        n["w_router"] = f + "router"
+        for x in ("up", "down"):
+            n[f"w_{x}_e"] = [f"{f}e{j}.{x}" for j in range(ls.moe.experts)]
+            if ls.moe.shared_ff:
+                n[f"w_{x}_s"] = f"{f}shared.{x}"
+    elif ls.ff:
+        n["w_gate"], n["w_up"], n["w_down"] = f + "gate", f + "up", f + "down"
+    return n
+
+
+def _migenex_shapes(ls, H: int) -> Dict[str, tuple]:
+    """What the config says about the shapes of a layer's logical tensors."""
+    s = {"w_in": (sum(_migenex_in_sizes(ls)), H), "w_o": (H, ls.heads * ls.vdim), "ln1_w": (H,), "ln1b_w": (H,), "ln2_w": (H,), "ln2b_w": (H,),
+         "q_norm_w": (ls.dim,), "k_norm_w": (ls.dim,), "w_gate": (ls.ff, H), "w_up": (ls.ff, H), "w_down": (H, ls.ff)}
+    if ls.moe is not None:
+        e = ls.moe
+        s.update({"w_router": (e.experts, H), "w_up_e": (e.experts, e.ff, H), "w_down_e": (e.experts, H, e.ff), "w_up_s": (e.shared_ff, H),
+                  "w_down_s": (H, e.shared_ff)})
+    return s
+
+
+def _migenex_in_sizes(ls) -> List[int]:
+    """Rows of the parts of w_in."""
+    return [ls.heads * ls.dim, ls.kv_heads * ls.dim] + ([] if ls.k_values else [ls.kv_heads * ls.vdim]) + ([ls.heads * ls.vdim] if ls.out_gate else [])
+
+
+def _load_migenex_weights(rd, spec: ModelSpec, plan: StagePlan, device, dtype) -> StageWeights:
+    w, H = StageWeights(spec, plan), spec.hidden_size
+    get = lambda name: rd.get(name).to(device=device, dtype=dtype)
+    w.embed, w.lm_head, w.final_norm_w = get("embed"), get("head"), get("final.norm")
+    want = {"embed": (w.embed, (spec.vocab_size, H)), "head": (w.lm_head, (spec.vocab_size, H)), "final.norm": (w.final_norm_w, (H,))}
+    if spec.bigram:
+        w.bigram = get("bigram")
+        want["bigram"] = (w.bigram, (spec.bigram[0] + 1, H))
+    if spec.loop_input:
+        w.loop_in = get("loop.in")
+        want["loop.in"] = (w.loop_in, (H, 2 * H))
+    for k, (t, shape) in want.items():
+        if tuple(t.shape) != shape:
+            raise ValueError(f"{k} has the shape {tuple(t.shape)}, the config says {shape}")
+    for i in plan.layers:
+        ls, l = spec.layer_specs[i], {}
+        shapes = _migenex_shapes(ls, H)
+        for k, names in _migenex_layer_names(ls, f"l{i}.").items():
+            if isinstance(names, tuple):
+                l[k] = torch.cat([get(x) for x in names], dim=0)
+            elif isinstance(names, list):
+                l[k] = torch.stack([get(x) for x in names], dim=0)
+            else:
+                l[k] = get(names)
+            if tuple(l[k].shape) != shapes[k]:
+                raise ValueError(f"layer {i}: {k} has the shape {tuple(l[k].shape)}, the config says {shapes[k]}")
+        w.layers.append(l)
+    return w
+
+
+def export_migenex_state_dict(w: StageWeights) -> Dict[str, torch.Tensor]:
+    """Logical -> checkpoint names (tests, `save` of random models)."""
+    sd = {"embed": w.embed, "head": w.lm_head, "final.norm": w.final_norm_w}
+    if w.bigram is not None:
+        sd["bigram"] = w.bigram
+    if w.loop_in is not None:
+        sd["loop.in"] = w.loop_in
+    for i, l in zip(w.plan.layers, w.layers):
+        ls = w.spec.layer_specs[i]
+        for k, names in _migenex_layer_names(ls, f"l{i}.").items():
+            if isinstance(names, tuple):
+                sd.update(zip(names, torch.split(l[k], _migenex_in_sizes(ls))))
+            elif isinstance(names, list):
+                sd.update(zip(names, l[k]))
+            else:
+                sd[names] = l[k]
+    return {k: v.detach().clone().contiguous() for k, v in sd.items()}
+
+
+def _random_migenex_weights(spec: ModelSpec, plan: StagePlan, seed: int, device, dtype) -> StageWeights:
+    """Random weights with which every mechanism matters: projections at 1 / sqrt(fan-in), norm weights around one, a bigram
+    table as large as the scaled embedding, a pass map that keeps half of the stream and of the embedding output."""
+    H, V = spec.hidden_size, spec.vocab_size
+    w = StageWeights(spec, plan)
+    rn = lambda name, shape, std: _randn(name, shape, seed, device, dtype, std=std)
+    one = lambda name, shape, std: torch.ones(shape, device=device, dtype=dtype) + rn(name, shape, std)
+    w.embed, w.lm_head, w.final_norm_w = rn("embed", (V, H), 1.0 / max(spec.embed_scale, 1e-6)), rn("head", (V, H), H ** -0.5), one("final.norm", (H,), 0.1)
+    if spec.bigram:
+        w.bigram = rn("bigram", (spec.bigram[0] + 1, H), 0.7)
+    if spec.loop_input:
+        w.loop_in = rn("loop.in", (H, 2 * H), (2 * H) ** -0.5)
+    for i in plan.layers:
+        ls, p, l = spec.layer_specs[i], f"layers.{i}.", {}
+        for k, shape in _migenex_shapes(ls, H).items():
+            if k not in _migenex_layer_names(ls, p):
+                continue
+            l[k] = one(p + k, shape, 0.15) if len(shape) == 1 else rn(p + k, shape, {"w_router": 2.0}.get(k, 1.0) * shape[-1] ** -0.5)
+        w.layers.append(l)
+    return w
+
+
 def _random_hybrid_weights(spec: ModelSpec, plan: StagePlan, seed: int, device, dtype) -> StageWeights:
     """Random weights of a hybrid stack, scaled so that activations stay of order one through any depth
     (projections at 1 / sqrt(fan-in), embedding at one) and every bias, convolution tap and gate matters."""
@@ -619,6 +734,8 @@ def _random_hybrid_weights(spec: ModelSpec, plan: StagePlan, seed: int, device, 
         return _random_zovozen_weights(spec, plan, seed, device, dtype)
     if spec.family == "pifutar":
         return _random_pifutar_weights(spec, plan, seed, device, dtype)
+    if spec.family == "migenex":
+        return _random_migenex_weights(spec, plan, seed, device, dtype)
     H, V = spec.hidden_size, spec.vocab_size
     w = StageWeights(spec, plan)
     rn = lambda name, shape, std: _randn(name, shape, seed, device, dtype, std=std)
@@ -660,6 +777,8 @@ def _load_hybrid_weights(rd, spec: ModelSpec, plan: StagePlan, device, dtype) ->
         return _load_zovozen_weights(rd, spec, plan, device, dtype)
     if spec.family == "pifutar":
         return _load_pifutar_weights(rd, spec, plan, device, dtype)
+    if spec.family == "migenex":
+        return _load_migenex_weights(rd, spec, plan, device, dtype)
     w = StageWeights(spec, plan)
     get = lambda name: rd.get(name).to(device=device, dtype=dtype)
     if plan.has_embed or plan.has_head:
