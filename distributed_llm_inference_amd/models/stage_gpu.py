@@ -434,8 +434,8 @@ class GpuStage:
         ok = [s for s in slots if 0 <= s < self.max_slots]
         self._write_table_rows(ok, [[]] * len(ok))
 
-    def _embed_rows(self, wk, T: int, ids, pos):
-        """wk.h[:T] <- embedding rows of `ids` (plus the learned position rows where the family has them)."""
+    def _embed_rows(self, wk, T: int, ids, pos, seq):
+        """wk.h[:T] <- embedding rows of `ids` (plus the learned position rows where the family has them). `seq`: the tokens' slots."""
         self.K.embed(wk.h[:T], ids, pos, self.embed, self.pos_embed)
 
     # ---- the layer stack on T tokens ------------------------------------------------------
@@ -617,7 +617,7 @@ class GpuStage:
                 ids = x.to(dtype=torch.int32).reshape(-1)
                 if ids.numel() != T:
                     raise ValueError(f"expected {T} token ids, got {ids.numel()}")
-            self._embed_rows(wk, T, ids, md_tok_pos)
+            self._embed_rows(wk, T, ids, md_tok_pos, md_tok_seq)
         else:
             if tuple(x.shape) != (T, s.hidden_size):
                 raise ValueError(f"expected hidden [{T},{s.hidden_size}], got {tuple(x.shape)}")
@@ -701,7 +701,7 @@ class GpuStage:
         """One decode step over the micro-batch's static buffers (captured into the graph)."""
         K, B, wk = self.K, st.B, st.wk
         if self.plan.has_embed:
-            self._embed_rows(wk, B, st.ids, st.ctx)
+            self._embed_rows(wk, B, st.ids, st.ctx, st.slots)
         else:
             wk.h[:B].copy_(st.hidden_in)
         pend = self._layers(wk, B, B, st.ctx, st.slots, self._arange[:B + 1], st.ctx, st.slots, 1, st.splits)

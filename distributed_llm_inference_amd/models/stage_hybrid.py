@@ -68,6 +68,17 @@ Stacks with convolved sublayer inputs and a learned average over depth (`spec.in
                   layers);  shared gate | up | sigmoid gate GEMM -> activation -> shared down GEMM ]
              -> join (x += experts + shared, kept as X_(i+1), x <- sum_j c_j X_j, the next layer's factor and input)
 
+Stacks with plain-weight norms on both sides of every sublayer (`spec.sandwich`; a stretch of layers may run several times, every
+pass behind a linear map of the stream beside the embedding output) run through `_layers_sand`: per layer run
+
+    x (fp32) -> norm -> ONE input GEMM (all projections of the mixer)
+             -> per-head norms + rotation + cache write (one kernel; the values may be the keys as projected)
+             -> attention (window, capped scores, entry gate) -> o GEMM -> join (x += m rms(y) w, and the next norm: one kernel)
+             -> [ gate | up GEMM -> relu(gate) * up -> down GEMM
+                | router | shared up GEMM -> route -> plan -> the experts' GEMMs over sorted rows, their inputs weighted;
+                  squared relu -> shared down GEMM ]
+             -> join (x += m rms(experts + shared) w, and the next norm, or the stream in the pass map's input -> map GEMM -> norm)
+
 Matrix products take bf16 operands (or fp32: `dtype="fp32"`, everything in true 32-bit) and accumulate in
 fp32; norms, scores, softmax, value mixing, gates, decays and states are fp32 in both modes.
 """
@@ -161,7 +172,11 @@ class HybridGpuStage(GpuStage):
         self.mfma_attn = [mfma_ok and ls.kind == "attention" and ls.dim == ls.vdim and ls.dim in (64, 128) and ls.group <= 16
                           for ls in self.specs]
         self._no_rope = {D: torch.zeros(1, D // 2, device=self.device) for D in (64, 128)}
-        if spec.norm_kind == "dyt":
+        if spec.sandwich:
+            # one cache per layer RUN
+            self._attn_of_run = [spec.layer_specs[li] for li, _ in spec.layer_runs()]
+            self.mfma_attn = [mfma_ok and a.dim == a.vdim and a.dim in (64, 128) and a.group <= 16 for a in self._attn_of_run]
+        elif spec.norm_kind == "dyt":
             # one cache / state per layer RUN
             self._attn_of_run = [spec.layer_specs[li].branches[0] if spec.layer_specs[li].kind == "parallel" else None for li, _ in spec.layer_runs()]
             self.mfma_attn = [mfma_ok and a is not None and a.dim == a.vdim and a.dim in (64, 128) and a.group <= 16 for a in self._attn_of_run]
@@ -171,7 +186,14 @@ class HybridGpuStage(GpuStage):
         self.par = spec.parallel_block
         self.post = spec.post_norm
         self.canon = spec.input_conv > 0 or spec.depth_average
+        self.sand = spec.sandwich
         self.runs = spec.layer_runs()
+        if self.sand:
+            # layers of other sizes: the tile kernel in bf16 where a head's query and key come in whole 16-byte pieces, else, and in
+            # fp32, the one-wave-per-(token, head) kernel. DLIA_SAND_TILE_ATTN=0: all of those on the latter (A/B)
+            tile_ok = dtype == "bf16" and os.environ.get("DLIA_SAND_TILE_ATTN", "1") != "0"
+            self._tile = [tile_ok and a.dim % 8 == 0 for a in self._attn_of_run]
+            self._load_sand(weights, f32, mat)
         if self.canon:
             self.mfma_attn = [False] * len(self.specs)
             # attention over the latent rows on the matrix cores in bf16 where the row and the latent come in whole 16-byte pieces;
@@ -197,7 +219,7 @@ class HybridGpuStage(GpuStage):
                             bool(self.K.mixed_attention_fits(a.heads, a.kv_heads, a.dim, a.vdim))
                             for a, tile in zip(self._attn_of_run, self._tile)]
             self._load_post(weights, f32, mat)
-        if self.post or self.canon:
+        if self.post or self.canon or self.sand:
             pass
         elif self.par:
             self.mfma_attn = [False] * len(self.specs)
@@ -285,7 +307,7 @@ class HybridGpuStage(GpuStage):
                 b = ls.branches[1]
                 self.rec.append((torch.zeros(max_slots + 1, b.heads, b.dim, b.vdim + 1, device=dev),
                                  torch.zeros(max_slots + 1, b.heads, 128, device=dev)))
-        for ls in ([] if (self.gated or self.par or self.post or self.canon) else self.specs):
+        for ls in ([] if (self.gated or self.par or self.post or self.canon or self.sand) else self.specs):
             if ls.kind == "delta":
                 C = 2 * ls.kv_heads * ls.dim + ls.heads * ls.vdim
                 self.rec.append((torch.zeros(max_slots + 1, max(ls.conv - 1, 1), C, device=dev),
@@ -340,6 +362,8 @@ class HybridGpuStage(GpuStage):
 
     # ---- workspaces ---------------------------------------------------------------------------------------
     def _new_work(self, rows: int):
+        if self.sand:
+            return self._new_work_sand(rows)
         if self.canon:
             return self._new_work_canon(rows)
         if self.post:
@@ -379,11 +403,12 @@ class HybridGpuStage(GpuStage):
         e = 4 if self.act_dtype == torch.float32 else 2
         if self.par or self.canon:
             return max(1, sum(BLOCK * e * sum(self._par_rows(li)) for li, ls in enumerate(self.specs) if self._keeps_rows(ls)))
-        return max(1, sum(ls.kv_heads * BLOCK * (ls.dim + ls.vdim) * e for ls in self._attn_of_run if ls is not None))
+        ids = 4 * BLOCK if self.spec.bigram else 0            # (the page of token ids)
+        return max(1, ids + sum(ls.kv_heads * BLOCK * (ls.dim + ls.vdim) * e for ls in self._attn_of_run if ls is not None))
 
     def _decode_state_bytes(self) -> int:
         n = 0
-        if self.gated or self.par or self.post or self.canon:
+        if self.gated or self.par or self.post or self.canon or self.sand:
             per_row = sum(t.numel() * t.element_size() for t in vars(self.wk0).values() if torch.is_tensor(t)) // self.max_tokens
             return sum(B * (per_row + 4 * self.vocab_pad) for B in self.graph_sizes)
         for B in self.graph_sizes:
@@ -395,6 +420,18 @@ class HybridGpuStage(GpuStage):
     def allocate_kv(self, num_blocks: int):
         dev, at = self.device, self.act_dtype
         self.num_blocks = int(num_blocks)
+        if self.sand:
+            self.id_pages = torch.zeros(self.num_blocks, BLOCK, device=dev, dtype=torch.int32) if self.spec.bigram else None
+            self.kv = []
+            for a, fast, tile in zip(self._attn_of_run, self.mfma_attn, self._tile):
+                G = a.kv_heads
+                if fast:              # K and V slabs of a block side by side, in fragment order
+                    self.kv.append(torch.zeros(self.num_blocks, G, 2, BLOCK * a.dim, device=dev, dtype=at))
+                    continue
+                kc = torch.zeros(self.num_blocks, G, BLOCK, a.dim, device=dev, dtype=at)
+                vc = torch.zeros(self.num_blocks, G, *((a.vdim, BLOCK) if tile else (BLOCK, a.vdim)), device=dev, dtype=at)
+                self.kv.append((kc, vc))
+            return
         if self.post:
             # keys: with the head mix folded into the query every head reads ALL key heads, so a token's keys are one row;
             # values per key / value head, key-contiguous where the matrix-core kernel reads them
@@ -447,7 +484,13 @@ class HybridGpuStage(GpuStage):
             st.slots.copy_(saved)
 
     # ---- the layer stack ----------------------------------------------------------------------------------
-    def _embed_rows(self, wk, T: int, ids, pos):
+    def _embed_rows(self, wk, T: int, ids, pos, seq):
+        if self.sand:
+            s = self.spec
+            _, mul_prev, mul_cur = s.bigram or (1, 0, 0)
+            self.K.embed_bigram(wk.h[:T], wk.cat[:T] if s.loop_input else None, s.loop_input and s.loop[0] == 0, ids, self.embed, s.embed_scale,
+                                self.bigram, mul_prev, mul_cur, self.id_pages, pos, seq, self.block_table)
+            return
         if self.canon:
             self.K.embed32(wk.hist[0][:T], ids, self.embed)
             if self._plan_rows:
@@ -461,6 +504,8 @@ class HybridGpuStage(GpuStage):
 
     def _layers(self, wk: _HybridWork, T: int, B: int, tok_pos, tok_seq, q_start, ctx, slots, max_q: int, splits: int,
                 alone: bool = False, lead_decode: int = 0):
+        if self.sand:
+            return self._layers_sand(wk, T, B, tok_pos, tok_seq, q_start, ctx, slots, max_q, lead_decode)
         if self.canon:
             return self._layers_canon(wk, T, B, tok_pos, tok_seq, q_start, ctx, slots, max_q)
         if self.post:
@@ -1355,6 +1400,181 @@ class HybridGpuStage(GpuStage):
                 self.layer_outputs.append(h.clone())
         return None
 
+    # ---- stacks with plain-weight norms on both sides of every sublayer -----------------------------------------------------
+    def _load_sand(self, weights: StageWeights, f32, mat):
+        """Device weights of the stack. A mixer's input projections are ONE matrix, the dense gate | up another, the router and the
+        shared expert's up projection a third. The residual multiplier rides in the weights of the norms behind the sublayers
+        (fp32); norm weights and rotation tables are fp32 in both modes."""
+        from .rope import rope_table
+        spec, dev, H = self.spec, self.device, self.spec.hidden_size
+        if H > int(self.K.sandwich_join_max_width(H % 4 == 0)):
+            raise ValueError(f"width {H} is beyond what the row kernels take")
+        self.embed, self.pos_embed, self.lm_head, self.lm_head_p = mat(weights.embed), None, mat(weights.lm_head), None
+        self.bigram = mat(weights.bigram) if spec.bigram else None
+        self.id_pages = None
+        self.final_norm_w = f32(weights.final_norm_w)
+        self.vocab_pad = packing.padded_n(spec.vocab_size)
+        self.loop_p: Dict[str, object] = {}
+        if spec.loop_input:
+            self._matrix(self.loop_p, "w_loop", mat(weights.loop_in), None)
+        self.layers = []
+        tables: Dict[tuple, tuple] = {}
+        for i, ls in enumerate(self.specs):
+            l = weights.layers[i]
+            p: Dict[str, object] = {"ln1_w": f32(l["ln1_w"]), "ln1b_w": (f32(l["ln1b_w"]) * spec.residual_mult).contiguous()}
+            self._matrix(p, "w_in", mat(l["w_in"]), None)
+            self._matrix(p, "w_o", mat(l["w_o"]), None)
+            p["q_norm_w"], p["k_norm_w"] = (f32(l["q_norm_w"]), f32(l["k_norm_w"])) if ls.head_norm else (None, None)
+            p["cos"] = p["sin"] = None
+            if ls.rope_dims:
+                key = (ls.rope_dims, ls.rope_base, ls.rope_scaling)
+                if key not in tables:
+                    tables[key] = tuple(t.contiguous() for t in rope_table(ls.rope_dims, ls.rope_base, ls.rope_scaling, self.max_seq_len, dev))
+                p["cos"], p["sin"] = tables[key]
+            if ls.has_ff:
+                p["ln2_w"], p["ln2b_w"] = f32(l["ln2_w"]), (f32(l["ln2b_w"]) * spec.residual_mult).contiguous()
+            if ls.moe is not None:
+                e = ls.moe
+                if e.outputs > 256:
+                    raise ValueError(f"layer {i}: up to 256 experts are supported")
+                self._matrix(p, "w_ff", torch.cat([mat(l["w_router"])] + ([mat(l["w_up_s"])] if e.shared_ff else [])), None)
+                p["w_up_e"], p["w_down_e"] = mat(l["w_up_e"]), mat(l["w_down_e"])
+                if e.shared_ff:
+                    self._matrix(p, "w_down_s", mat(l["w_down_s"]), None)
+            elif ls.ff:
+                self._matrix(p, "w_gu", torch.cat([mat(l["w_gate"]), mat(l["w_up"])]), None)
+                self._matrix(p, "w_down", mat(l["w_down"]), None)
+            self.layers.append(p)
+            weights.layers[i] = {}
+        if self._packed and H % 128 == 0:
+            self.lm_head_p = packing.pack_weight(self.lm_head)
+            self._shapes.append((self.vocab_pad, H, False))
+
+    def _new_work_sand(self, rows: int):
+        s, dev, at = self.spec, self.device, self.act_dtype
+        z = lambda n, dt=torch.float32: torch.zeros(max(int(n), 1), device=dev, dtype=dt)
+        B, H = min(rows, self.max_batch), s.hidden_size
+        zc = z16 = qc = q16 = mc = yc = z2 = gu = ac = part = 1
+        pairs = tiles = ef = 0
+        for (li, _), fast, tile in zip(self.runs, self.mfma_attn, self._tile):
+            a, p = self.specs[li], self.layers[li]
+            zc, z16 = (zc, max(z16, self._cols(p, "w_in"))) if fast else (max(zc, self._cols(p, "w_in")), z16)
+            qc, q16 = (qc, max(q16, a.heads * a.dim)) if fast or tile else (max(qc, a.heads * a.dim), q16)
+            if tile and not fast:
+                part = max([part] + [int(self.K.tile_attention_part_floats(b, a.heads, a.kv_heads, a.vdim, 1)) for b in range(1, B + 1)])
+        for ls, p in zip(self.specs, self.layers):
+            mc, yc = max(mc, ls.heads * ls.vdim), max(yc, self._cols(p, "w_o"))
+            if ls.moe is not None:
+                e = ls.moe
+                z2 = max(z2, self._cols(p, "w_ff"))
+                # (rows of the experts' sorted copies: whole tiles of 32 rows, or of 128 for steps with many rows)
+                pairs, ef = max(pairs, rows * e.top), max(ef, e.ff)
+                tiles = max(tiles, (rows * e.top + 31) // 32 + e.experts, 4 * ((rows * e.top + 127) // 128 + e.experts))
+                if e.shared_ff:
+                    ac, yc = max(ac, e.shared_ff), max(yc, self._cols(p, "w_down_s"))
+            elif ls.ff:
+                gu, ac, yc = max(gu, self._cols(p, "w_gu")), max(ac, ls.ff), max(yc, self._cols(p, "w_down"))
+        ws_floats = self._ws_floats
+        if self._packed and rows > self.decode_rows:
+            for m_ in {rows, min(rows, 512), min(rows, 1024)}:
+                if m_ > self.decode_rows:
+                    ws_floats = max([ws_floats] + [int(self.K.gemm_ws_floats(m_, n_, k_)) for n_, k_, _ in self._shapes])
+        i32 = torch.int32
+        return SimpleNamespace(
+            h=torch.zeros(rows, H, device=dev), xn=torch.zeros(rows, H, device=dev, dtype=at),
+            cat=torch.zeros(rows if s.loop_input else 1, 2 * H, device=dev, dtype=at), z=z(rows * zc), z16=z(rows * z16, torch.bfloat16),
+            q32=z(rows * qc), q16=z(rows * q16, torch.bfloat16), mixed=z(rows * mc, at), ya=z(rows * yc), z2=z(rows * z2), gu=z(rows * gu, at),
+            act=z(rows * ac, at), sel=z(pairs, i32), wts=z(pairs), pair_row=z(pairs, i32), tiles=z(1 + tiles, i32), row_tok=z(32 * tiles, i32),
+            row_w=z(32 * tiles), eact=z(32 * tiles * ef, at), ey=z(32 * tiles * H), part=z(part), ws=z(ws_floats + 4096),
+            head_x=torch.zeros(B, H, device=dev, dtype=at), logits=torch.zeros(B, self.vocab_pad, device=dev), cmax=None, guided=False)
+
+    def _layers_sand(self, wk, T: int, B: int, tok_pos, tok_seq, q_start, ctx, slots, max_q: int, lead_decode: int):
+        K, spec, eps, H = self.K, self.spec, self.spec.norm_eps, self.spec.hidden_size
+        h, xn = wk.h[:T], wk.xn[:T]
+        view = lambda buf, cols: buf[:T * cols].view(T, cols)
+        keep = self.keep_layer_outputs and not torch.cuda.is_current_stream_capturing()
+        if keep:
+            self.layer_outputs = []
+        table, runs = self.block_table, self.runs
+        first = spec.loop[0] if spec.loop_input else -1
+        opens = lambda ri: ri < len(runs) and runs[ri][1] >= 0 and runs[ri][0] == first         # the run starts a pass
+
+        def enter(ri):
+            """The stream, in the map's input type, becomes the pass's first stream; its norm is what run ri reads."""
+            self._mm(wk, h, wk.cat[:T], self.loop_p, "w_loop")
+            K.sandwich_join(xn, h, None, None, None, None, 1, None, self.layers[runs[ri][0]]["ln1_w"], eps)
+
+        def join(wb, wn, follows, ya=None, yb=None, ey=None, top=1):
+            """Adds a sublayer's output; `wn`: the norm of the sublayer that reads next, else the run `follows` does."""
+            out = xn
+            if wn is None and follows is not None:
+                out = None if follows >= len(runs) else wk.cat[:T, :H] if opens(follows) else xn
+                wn = self.layers[runs[follows][0]]["ln1_w"] if out is xn else None
+            K.sandwich_join(out, h, ya, yb, ey, wk.pair_row if ey is not None else None, top, wb, wn, eps)
+
+        if opens(0):
+            enter(0)             # (the embedding left the stream in both halves of the map's input)
+        else:
+            K.sandwich_join(xn, h, None, None, None, None, 1, None, self.layers[runs[0][0]]["ln1_w"], eps)
+        for ri, (li, _) in enumerate(runs):
+            ls, p = self.specs[li], self.layers[li]
+            Hh, G, d, dv, fast, tile = ls.heads, ls.kv_heads, ls.dim, ls.vdim, self.mfma_attn[ri], self._tile[ri]
+            z = view(wk.z16 if fast else wk.z, self._cols(p, "w_in"))
+            self._mm(wk, z, xn, p, "w_in")
+            q, mixed = view(wk.q16 if fast or tile else wk.q32, Hh * d), view(wk.mixed, Hh * dv)
+            kc, vc = (self.kv[ri], None) if fast else self.kv[ri]
+            col_v = -1 if ls.k_values else (Hh + G) * d
+            c_g = (Hh + G) * d + (0 if ls.k_values else G * dv)
+            gate = z[:, c_g:c_g + Hh * dv] if ls.out_gate else None
+            K.qk_prep(z, Hh, G, d, dv, col_v, p["q_norm_w"], p["k_norm_w"], ls.unit_qk, eps, ls.rope_dims, ls.rope_interleaved, p["cos"], p["sin"],
+                      q, kc, vc, 2 if fast else 1 if tile else 0, tok_pos, tok_seq, table)
+            # single tokens riding in front of prompt portions: the decode-shaped kernel for them, the prefill-shaped for the rest
+            n = lead_decode if (fast or tile) and 0 < lead_decode < B and max_q > 1 else 0
+            for b0, b1, mq, r1 in ([(0, n, 1, n)] if n else []) + [(n, B, max_q, T)]:
+                win = ls.window or 0
+                if fast:
+                    K.paged_attention_capped(mixed, q, kc, q_start[b0:b1 + 1], ctx[b0:b1], table, slots[b0:b1], mq, Hh, G, d, ls.scale, win,
+                                             ls.softcap, gate)
+                elif tile:
+                    K.tile_attention(mixed[:r1], q[:r1], d, kc, vc, q_start[b0:b1 + 1], ctx[b0:b1], slots[b0:b1], table, mq, Hh, d, dv, 1, ls.scale,
+                                     win, 0, ls.softcap, 0.0, 1.0, eps, gate[:r1] if gate is not None else None, wk.part)
+                else:
+                    K.multi_attention(mixed, q, d, kc, vc, 0, tok_pos, tok_seq, table, Hh, d, dv, 1, ls.scale, win, 0, ls.softcap, 0.0, 1.0, eps, gate)
+            ya = view(wk.ya, self._cols(p, "w_o"))
+            self._mm(wk, ya, mixed, p, "w_o")
+            join(p["ln1b_w"], p["ln2_w"] if ls.has_ff else None, ri + 1, ya[:, :H])
+            if ls.moe is not None:
+                e = ls.moe
+                z2 = view(wk.z2, self._cols(p, "w_ff"))
+                self._mm(wk, z2, xn, p, "w_ff")
+                # row tiles: 128 rows through the LDS-tiled kernel when the step has many rows (bf16, inner sizes in whole
+                # k-steps), else 32 rows through the register-tiled kernels; at most nt tiles hold a row
+                tr = 128 if (self.wmode == "bf16" and T * e.top >= 1024 and H % 32 == 0 and e.ff % 32 == 0) else 32
+                nt = (T * e.top + tr - 1) // tr + e.experts
+                eact, ey = wk.eact[:tr * nt * e.ff].view(tr * nt, e.ff), wk.ey[:tr * nt * H].view(tr * nt, H)
+                K.moe_route(wk.sel, wk.wts, z2[:, :e.outputs], e.top, e.groups, e.keep, e.scale, None, e.score == "softmax", e.group_rank, e.renorm)
+                K.moe_plan(wk.tiles, wk.row_tok, wk.pair_row, wk.sel, T * e.top, e.top, e.experts, tr, wk.wts, wk.row_w)
+                K.moe_up(eact, xn, None, p["w_up_e"], wk.tiles, wk.row_tok, nt, 0.0, tr, wk.row_w)
+                K.moe_down(ey, eact, p["w_down_e"], wk.tiles, wk.row_tok, nt, tr)
+                yb = None
+                if e.shared_ff:
+                    act, yb = view(wk.act, e.shared_ff), view(wk.ya, self._cols(p, "w_down_s"))
+                    K.relu_act(act, z2[:, e.outputs:e.outputs + e.shared_ff], False)
+                    self._mm(wk, yb, act, p, "w_down_s")
+                    yb = yb[:, :H]
+                join(p["ln2b_w"], None, ri + 1, None, yb, ey, e.top)
+            elif ls.ff:
+                gu, act, ya = view(wk.gu, self._cols(p, "w_gu")), view(wk.act, ls.ff), view(wk.ya, self._cols(p, "w_down"))
+                self._mm(wk, gu, xn, p, "w_gu")
+                K.relu_act(act, gu, True)
+                self._mm(wk, ya, act, p, "w_down")
+                join(p["ln2b_w"], None, ri + 1, ya[:, :H])
+            if keep:
+                self.layer_outputs.append(h.clone())
+            if opens(ri + 1):
+                enter(ri + 1)
+        return None
+
     def _fold(self, wk, T: int, pend):
         return None
 
@@ -1364,7 +1584,7 @@ class HybridGpuStage(GpuStage):
         if self.gated:
             K.dyt_gate(hx, wk.h[:T], None, None, None, None, None, None, None, self.final_norm_w, self.final_norm_b, rows_idx[:R],
                        self.final_norm_a, self.spec.norm_eps)
-        elif self.par or self.post:
+        elif self.par or self.post or self.sand:
             K.norm32(hx, wk.h[:T], None, None, self.final_norm_w, rows_idx[:R], self.spec.norm_eps, 0.0)
         else:
             K.norm32(hx, wk.h[:T], None, None, self.final_norm_w, rows_idx[:R], self.spec.norm_eps, 1.0)

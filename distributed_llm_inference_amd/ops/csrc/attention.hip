@@ -64,15 +64,35 @@ struct AttnParams {
   // `gate` [T, ldg]: the head's output is multiplied by sigmoid(gate[row, head]).
   const float* temp; const float* bias; const float* sinkv; const float* gate;
   int bias_rows; long ldg;
+  // Capped / entry-gated instantiations (EXT 2: the window, none of the extras above): `cap` > 0: a score s (in the units of
+  // q . k) becomes cap tanh(s * inv_cap), cap and inv_cap carrying the softmax scale; `egate` [T, lde] bf16: every entry of a
+  // head's output is multiplied by the sigmoid of its own logit.
+  float cap, inv_cap;
+  const bf16* egate; long lde;
 };
+
+// tanh in fp32 from the hardware exponential: 1 - 2 / (exp(2 y) + 1); large |y| saturate to +-1 by themselves.
+__device__ __forceinline__ float tanh_exp(float y) {
+  return 1.f - 2.f * __builtin_amdgcn_rcpf(__builtin_amdgcn_exp2f(y * 2.8853900817779268f) + 1.f);
+}
+// acc[r] *= sigmoid(gate[r]) for four neighbouring entries
+__device__ __forceinline__ f32x4 entry_gate(const bf16* g, f32x4 acc) {
+  const u32x2 v = *reinterpret_cast<const u32x2*>(g);
+  const float z[4] = {bf16_lo(v.x), bf16_hi(v.x), bf16_lo(v.y), bf16_hi(v.y)};
+#pragma unroll
+  for (int r = 0; r < 4; ++r) acc[r] *= 1.f / (1.f + __expf(-z[r]));
+  return acc;
+}
 
 constexpr float kNegInf = -__builtin_inff();
 
 // NW = waves per work item: 4 interleave the item's KV blocks and merge at the end (few items, long
 // contexts); 1 walks all of them alone with no LDS and no barrier (decode over thousands of
 // (sequence, kv head) items, where a 160-token context is 5 blocks and 4 waves would take 2, 1, 1, 1).
-template <int D, int NT, bool KV8, int NW, bool PF, bool WIN = false>
+// EXT: 0 plain causal; 1 window, sink and the learned extras; 2 window, capped scores and the entry gate.
+template <int D, int NT, bool KV8, int NW, bool PF, int EXT = 0>
 __device__ __forceinline__ void paged_attn_body(const AttnParams& p, long item) {
+  constexpr bool WIN = EXT >= 1, LEARNED = EXT == 1, CAPPED = EXT == 2;
   constexpr int KS = D / 32;      // MFMA k-steps over the head dim (QK^T)
   constexpr int DT = D / 16;      // 16-row tiles of the head dim (PV)
   constexpr int NC = NT * 16;     // query columns per workgroup
@@ -112,7 +132,7 @@ __device__ __forceinline__ void paged_attn_body(const AttnParams& p, long item) 
   }
   [[maybe_unused]] float col_temp[NT], col_sink[NT];
   [[maybe_unused]] const float* col_bias[NT];
-  if constexpr (WIN) {
+  if constexpr (LEARNED) {
 #pragma unroll
     for (int nt = 0; nt < NT; ++nt) {
       const int hc = min(col_head[nt], p.Hq - 1);           // (padding columns stay inside the tables)
@@ -224,7 +244,15 @@ __device__ __forceinline__ void paged_attn_body(const AttnParams& p, long item) 
     for (int nt = 0; nt < NT; ++nt) {
       const int limit = col_qpos[nt] >= 0 ? ctx + col_qpos[nt] : -1;   // last visible key position
       float mx = kNegInf;
-      if constexpr (WIN) {
+      if constexpr (CAPPED) {
+        if (p.cap > 0.f) {
+#pragma unroll
+          for (int kt = 0; kt < 2; ++kt)
+#pragma unroll
+            for (int r = 0; r < 4; ++r) st[kt][nt][r] = p.cap * tanh_exp(st[kt][nt][r] * p.inv_cap);
+        }
+      }
+      if constexpr (LEARNED) {
         if (p.temp || p.bias) {
 #pragma unroll
           for (int kt = 0; kt < 2; ++kt)
@@ -311,16 +339,19 @@ __device__ __forceinline__ void paged_attn_body(const AttnParams& p, long item) 
       lt += __shfl_xor(lt, 16, 64);
       lt += __shfl_xor(lt, 32, 64);
       if (col_qpos[nt] < 0) continue;
-      if constexpr (WIN) {
+      if constexpr (LEARNED) {
         if (p.sink && p.splits == 1) lt += exp2f((col_sink[nt] - (m[nt] == kNegInf ? 0.f : m[nt])) * p.scale_log2);
       }
       float inv = lt > 0.f ? 1.f / lt : 0.f;
-      if constexpr (WIN) {
+      if constexpr (LEARNED) {
         if (p.gate) inv *= 1.f / (1.f + expf(-p.gate[col_row[nt] * p.ldg + col_head[nt]]));
       }
 #pragma unroll
       for (int dt = 0; dt < DT; ++dt) {
-        const f32x4 acc = o[dt][nt];
+        f32x4 acc = o[dt][nt];
+        if constexpr (CAPPED) {
+          if (p.egate) acc = entry_gate(p.egate + col_row[nt] * p.lde + col_head[nt] * D + dt * 16 + quad * 4, acc);
+        }
         if (p.splits == 1) {
           u32x2 v = {pack_bf16(acc[0] * inv, acc[1] * inv), pack_bf16(acc[2] * inv, acc[3] * inv)};
           *reinterpret_cast<u32x2*>(p.out + col_row[nt] * p.ldo + col_head[nt] * D + dt * 16 + quad * 4) = v;
@@ -367,17 +398,20 @@ __device__ __forceinline__ void paged_attn_body(const AttnParams& p, long item) 
       lt += lw[w] * wgt[w];
     }
     if (col_qpos[nt] < 0) continue;
-    if constexpr (WIN) {
+    if constexpr (LEARNED) {
       if (p.sink && p.splits == 1) lt += exp2f((col_sink[nt] - m_safe) * p.scale_log2);
     }
     float inv = lt > 0.f ? 1.f / lt : 0.f;
-    if constexpr (WIN) {
+    if constexpr (LEARNED) {
       if (p.gate) inv *= 1.f / (1.f + expf(-p.gate[col_row[nt] * p.ldg + col_head[nt]]));
     }
     for (int dt = wave; dt < DT; dt += 4) {
       f32x4 acc = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
       for (int w = 0; w < 4; ++w) acc += oacc[((w * DT + dt) * NT + nt) * 64 + lane] * wgt[w];
+      if constexpr (CAPPED) {
+        if (p.egate) acc = entry_gate(p.egate + col_row[nt] * p.lde + col_head[nt] * D + dt * 16 + quad * 4, acc);
+      }
       if (p.splits == 1) {
         u32x2 v = {pack_bf16(acc[0] * inv, acc[1] * inv), pack_bf16(acc[2] * inv, acc[3] * inv)};
         *reinterpret_cast<u32x2*>(p.out + col_row[nt] * p.ldo + col_head[nt] * D + dt * 16 + quad * 4) = v;
@@ -392,14 +426,14 @@ __device__ __forceinline__ void paged_attn_body(const AttnParams& p, long item) 
   }
 }
 
-template <int D, int NT, bool KV8, bool WIN = false>
-__global__ __launch_bounds__(256) void paged_attn_kernel(AttnParams p) { paged_attn_body<D, NT, KV8, 4, true, WIN>(p, blockIdx.x); }
+template <int D, int NT, bool KV8, int EXT = 0>
+__global__ __launch_bounds__(256) void paged_attn_kernel(AttnParams p) { paged_attn_body<D, NT, KV8, 4, true, EXT>(p, blockIdx.x); }
 
 // One wave per item, one block in flight per wave, registers capped so that 3 waves share a SIMD:
 // latency is hidden by the other waves instead of by a second set of K/V registers.
-template <int D, bool KV8, bool WIN = false>
+template <int D, bool KV8, int EXT = 0>
 __global__ __launch_bounds__(64) __attribute__((amdgpu_waves_per_eu(3, 4))) void paged_attn_lean_kernel(AttnParams p) {
-  paged_attn_body<D, 1, KV8, 1, false, WIN>(p, blockIdx.x);
+  paged_attn_body<D, 1, KV8, 1, false, EXT>(p, blockIdx.x);
 }
 
 // The same one-wave-per-item body in a fixed number of 4-wave workgroups (one wave per SIMD) that walk the item list
@@ -491,8 +525,9 @@ __device__ __forceinline__ float quad_sum(float x) {
   return __uint_as_float(b[0]) + __uint_as_float(b[1]);
 }
 
-template <int D, bool KV8, bool WIN = false>
+template <int D, bool KV8, int EXT = 0>
 __global__ __launch_bounds__(256, 2) void prefill_attn_kernel(AttnParams p) {
+  constexpr bool WIN = EXT >= 1, LEARNED = EXT == 1, CAPPED = EXT == 2;
   constexpr int KS = D / 32, DT = D / 16, NT = 2, NC = 128;
   constexpr int BLOCK_BYTES = 2 * 2 * kBlockTokens * D;               // K slab + V slab of one head as bf16 (in LDS)
   constexpr int MEM_BYTES = KV8 ? BLOCK_BYTES / 2 : BLOCK_BYTES;      // ... and as stored in the cache
@@ -552,7 +587,7 @@ __global__ __launch_bounds__(256, 2) void prefill_attn_kernel(AttnParams p) {
   }
   [[maybe_unused]] float col_temp[NT];
   [[maybe_unused]] const float* col_bias[NT];
-  if constexpr (WIN) {
+  if constexpr (LEARNED) {
 #pragma unroll
     for (int nt = 0; nt < NT; ++nt) {
       const int hc = min(kvh * p.g_real + ((wave * 32 + nt * 16 + l15) & (g - 1)), p.Hq - 1);
@@ -649,7 +684,15 @@ __global__ __launch_bounds__(256, 2) void prefill_attn_kernel(AttnParams p) {
 #pragma unroll
     for (int nt = 0; nt < NT; ++nt) {
       float mx = kNegInf;
-      if constexpr (WIN) {
+      if constexpr (CAPPED) {
+        if (p.cap > 0.f) {
+#pragma unroll
+          for (int kt = 0; kt < 2; ++kt)
+#pragma unroll
+            for (int r = 0; r < 4; ++r) st[kt][nt][r] = p.cap * tanh_exp(st[kt][nt][r] * p.inv_cap);
+        }
+      }
+      if constexpr (LEARNED) {
         if (p.temp || p.bias) {
           const int qabs = ctx + col_qpos[nt];
 #pragma unroll
@@ -763,22 +806,28 @@ __global__ __launch_bounds__(256, 2) void prefill_attn_kernel(AttnParams p) {
     asm volatile("" : "+v"(le));                   // recompute from the lane id instead of keeping the prologue's values live
     const int ce = wave * 32 + nt * 16 + (le & 15);
     [[maybe_unused]] const int he = kvh * p.g_real + (ce & (g - 1));
-    if constexpr (WIN) {
+    if constexpr (LEARNED) {
       if (p.sink) lt += exp2f(((p.sinkv ? p.sinkv[min(he, p.Hq - 1)] : 0.f) - (m[nt] == kNegInf ? 0.f : m[nt])) * p.scale_log2);
     }
     float inv = lt > 0.f ? 1.f / lt : 0.f;
-    if constexpr (WIN) {
+    if constexpr (LEARNED) {
       if (p.gate) inv *= 1.f / (1.f + expf(-p.gate[(long)(t0 + col_qpos[nt]) * p.ldg + he]));
     }
     bf16* orow = p.out + (long)(t0 + col_qpos[nt]) * p.ldo + (kvh * p.g_real + (ce & (g - 1))) * D + (le >> 4) * 4;
 #pragma unroll
     for (int dt = 0; dt < DT; ++dt) {
-      const f32x4 acc = o[dt][nt];
+      f32x4 acc = o[dt][nt];
+      if constexpr (CAPPED) {
+        if (p.egate) acc = entry_gate(p.egate + (long)(t0 + col_qpos[nt]) * p.lde + he * D + (le >> 4) * 4 + dt * 16, acc);
+      }
       u32x2 v = {pack_bf16(acc[0] * inv, acc[1] * inv), pack_bf16(acc[2] * inv, acc[3] * inv)};
       *reinterpret_cast<u32x2*>(orow + dt * 16) = v;
     }
   }
 }
+
+// scores with a cap or outputs with an entry gate: the EXT 2 instantiations
+static inline bool capped(const AttnParams& p) { return p.cap > 0.f || p.egate; }
 
 template <int D>
 static void launch_prefill_attn(const AttnParams& p, hipStream_t stream) {
@@ -786,7 +835,8 @@ static void launch_prefill_attn(const AttnParams& p, hipStream_t stream) {
   constexpr size_t smem = 2 * (4 * kBlockTokens * D + 256);      // two bf16 blocks + their scales
   const bool win = p.window > 0 || p.sink;
   if (p.kv_scale) hipLaunchKernelGGL((prefill_attn_kernel<D, true>), dim3((unsigned)nitems), dim3(256), smem, stream, p);
-  else if (win)   hipLaunchKernelGGL((prefill_attn_kernel<D, false, true>), dim3((unsigned)nitems), dim3(256), smem, stream, p);
+  else if (capped(p)) hipLaunchKernelGGL((prefill_attn_kernel<D, false, 2>), dim3((unsigned)nitems), dim3(256), smem, stream, p);
+  else if (win)   hipLaunchKernelGGL((prefill_attn_kernel<D, false, 1>), dim3((unsigned)nitems), dim3(256), smem, stream, p);
   else            hipLaunchKernelGGL((prefill_attn_kernel<D, false>), dim3((unsigned)nitems), dim3(256), smem, stream, p);
 }
 
@@ -806,11 +856,16 @@ static void launch_attn(const AttnParams& p, hipStream_t stream) {
   const long thr = wave_per_item_threshold();
   const char* pe = getenv("DLIA_ATTN_PERSIST");               // read per launch (a captured graph keeps what it was captured with)
   const long persist = pe ? atol(pe) : 0L;
-  if ((p.window > 0 || p.sink) && !p.kv_scale) {             // windowed / sink instantiations (bf16 cache)
+  if (capped(p) && !p.kv_scale) {                            // capped / entry-gated instantiations (bf16 cache)
     if (NT == 1 && thr > 0 && nitems >= thr)
-      hipLaunchKernelGGL((paged_attn_lean_kernel<D, false, true>), dim3((unsigned)nitems), dim3(64), 0, stream, p);
+      hipLaunchKernelGGL((paged_attn_lean_kernel<D, false, 2>), dim3((unsigned)nitems), dim3(64), 0, stream, p);
     else
-      hipLaunchKernelGGL((paged_attn_kernel<D, NT, false, true>), dim3((unsigned)nitems), dim3(256), smem, stream, p);
+      hipLaunchKernelGGL((paged_attn_kernel<D, NT, false, 2>), dim3((unsigned)nitems), dim3(256), smem, stream, p);
+  } else if ((p.window > 0 || p.sink) && !p.kv_scale) {      // windowed / sink instantiations (bf16 cache)
+    if (NT == 1 && thr > 0 && nitems >= thr)
+      hipLaunchKernelGGL((paged_attn_lean_kernel<D, false, 1>), dim3((unsigned)nitems), dim3(64), 0, stream, p);
+    else
+      hipLaunchKernelGGL((paged_attn_kernel<D, NT, false, 1>), dim3((unsigned)nitems), dim3(256), smem, stream, p);
   } else if (NT == 1 && thr > 0 && nitems >= thr && persist > 0 && nitems >= persist * 4 && !p.kv_scale) {
     hipLaunchKernelGGL((paged_attn_lean_persist_kernel<D, false>), dim3((unsigned)persist), dim3(256), 0, stream, p, nitems);
   } else if (NT == 1 && thr > 0 && nitems >= thr) {
@@ -863,10 +918,12 @@ extern "C" void dlia_paged_attention(void* out, const void* qkv, const void* kv_
                                      int Hkv, int D, int table_rows, int max_blocks, int num_blocks,
                                      long ldq, long ldo, float scale, int splits, hipStream_t stream, int window, int sink,
                                      const float* temp, const float* bias, int bias_rows, const float* sinkv, const float* gate,
-                                     long ldg) {
+                                     long ldg, float softcap, const void* egate, long lde) {
   if (B <= 0 || max_q_len <= 0) return;
   AttnParams p;
   p.window = kv_scale ? 0 : window; p.sink = kv_scale ? 0 : sink;
+  p.cap = softcap > 0.f && !kv_scale ? softcap / scale : 0.f; p.inv_cap = softcap > 0.f ? scale / softcap : 0.f;
+  p.egate = kv_scale ? nullptr : (const bf16*)egate; p.lde = lde;
   p.temp = temp; p.bias = bias; p.bias_rows = bias ? bias_rows : 1; p.sinkv = sinkv; p.gate = gate; p.ldg = ldg;
   p.out = (bf16*)out; p.ldo = ldo; p.q = (const bf16*)qkv; p.ldq = ldq; p.kv = (const bf16*)kv_cache; p.kv_scale = kv_scale;
   p.q_start = q_start; p.ctx_lens = ctx_lens; p.block_table = block_table; p.slots = slots; p.table_rows = table_rows; p.partial = partial;

@@ -446,7 +446,7 @@ static void paged_attention_impl(Tensor out, const Tensor& qkv, const Tensor& kv
                                  OptTensor slots, OptTensor partial, int64_t max_q_len, int64_t Hq, int64_t Hkv,
                                  int64_t D, double scale, int64_t splits, int64_t window = 0, bool sink = false,
                                  OptTensor temp = c10::nullopt, OptTensor bias = c10::nullopt, OptTensor sinkv = c10::nullopt,
-                                 OptTensor gate = c10::nullopt) {
+                                 OptTensor gate = c10::nullopt, double softcap = 0.0, OptTensor egate = c10::nullopt) {
   DLIA_ON_DEVICE_OF(out);
   check_bf16(out, "out"); check_bf16(qkv, "qkv"); check_rows(out, "out"); check_rows(qkv, "qkv");
   DLIA_CHECK(window >= 0 && (!kv_scale.has_value() || (window == 0 && !sink)), "window / sink: bf16 cache only, window >= 0");
@@ -496,13 +496,24 @@ static void paged_attention_impl(Tensor out, const Tensor& qkv, const Tensor& kv
       gp = gate->data_ptr<float>(); ldg = gate->stride(0);
     }
   }
+  const void* ep = nullptr; long lde = 0;
+  if (softcap > 0.0 || egate.has_value()) {
+    DLIA_CHECK(!sink && !tp && !bp && !sk && !gp && sp == 1 && !kv_scale.has_value() && scale > 0.0, "capped scores / entry gate: no sink or learned extras, no split, bf16 cache");
+    if (egate.has_value()) {
+      check_bf16(*egate, "egate");
+      DLIA_CHECK(egate->dim() == 2 && egate->stride(1) == 1 && egate->size(1) == Hq * D && egate->size(0) >= out.size(0) && egate->stride(0) % 4 == 0 &&
+                 reinterpret_cast<uintptr_t>(egate->data_ptr()) % 8 == 0, "entry gate logits: bf16 [T, Hq D] in aligned rows");
+      ep = egate->data_ptr(); lde = egate->stride(0);
+    }
+  }
   // The caller guarantees: q_start is non-decreasing with q_start[B] <= rows of qkv/out, chunk
   // lengths <= max_q_len, and ctx_lens[b] + q_len[b] <= 32 * block_table.size(1).
   dlia_paged_attention(out.data_ptr(), qkv.data_ptr(), kv_cache.data_ptr(),
                        kv_scale.has_value() ? kv_scale->data_ptr<float>() : nullptr, q_start.data_ptr<int>(),
                        ctx_lens.data_ptr<int>(), block_table.data_ptr<int>(), slp, pp, (int)B, (int)max_q_len, (int)Hq,
                        (int)Hkv, (int)D, (int)block_table.size(0), (int)block_table.size(1), (int)geo.num_blocks, qkv.stride(0),
-                       out.stride(0), (float)scale, sp, cur_stream(), (int)window, sink ? 1 : 0, tp, bp, brows, sk, gp, ldg);
+                       out.stride(0), (float)scale, sp, cur_stream(), (int)window, sink ? 1 : 0, tp, bp, brows, sk, gp, ldg,
+                       (float)softcap, ep, lde);
 }
 
 // Causal attention restricted to a sliding window (0: none), optionally with a softmax sink, over the bf16 cache.
@@ -521,6 +532,15 @@ void paged_attention_biased(Tensor out, const Tensor& qkv, const Tensor& kv_cach
                             double scale, OptTensor temp, OptTensor bias, OptTensor sinkv, OptTensor gate) {
   paged_attention_impl(out, qkv, kv_cache, c10::nullopt, q_start, ctx_lens, block_table, slots, c10::nullopt, max_q_len, Hq, Hkv, D,
                        scale, 1, 0, true, temp, bias, sinkv, gate);
+}
+
+// A window (0: none), scores through cap tanh(score / cap) (0: as they are), every entry of the output times the sigmoid of its
+// logit in `gate` [T, Hq D].
+void paged_attention_capped(Tensor out, const Tensor& q, const Tensor& kv_cache, const Tensor& q_start, const Tensor& ctx_lens,
+                            const Tensor& block_table, OptTensor slots, int64_t max_q_len, int64_t Hq, int64_t Hkv, int64_t D, double scale,
+                            int64_t window, double softcap, OptTensor gate) {
+  paged_attention_impl(out, q, kv_cache, c10::nullopt, q_start, ctx_lens, block_table, slots, c10::nullopt, max_q_len, Hq, Hkv, D, scale, 1,
+                       window, false, c10::nullopt, c10::nullopt, c10::nullopt, c10::nullopt, softcap, gate);
 }
 
 void value_mix(Tensor qkv, Tensor vfirst, OptTensor lam, int64_t mix, int64_t v_off, int64_t v_cols) {
@@ -883,6 +903,7 @@ TORCH_LIBRARY(dlia, m) {
   m.def("gated_gelu(Tensor(a!) act, Tensor gu) -> ()");
   m.def("paged_attention_window(Tensor(a!) out, Tensor qkv, Tensor kv_cache, Tensor q_start, Tensor ctx_lens, Tensor block_table, Tensor? slots, Tensor? partial, int max_q_len, int Hq, int Hkv, int D, float scale, int splits, int window, bool sink) -> ()");
   m.def("paged_attention_biased(Tensor(a!) out, Tensor qkv, Tensor kv_cache, Tensor q_start, Tensor ctx_lens, Tensor block_table, Tensor? slots, int max_q_len, int Hq, int Hkv, int D, float scale, Tensor? temp, Tensor? bias, Tensor? sinkv, Tensor? gate) -> ()");
+  m.def("paged_attention_capped(Tensor(a!) out, Tensor q, Tensor kv_cache, Tensor q_start, Tensor ctx_lens, Tensor block_table, Tensor? slots, int max_q_len, int Hq, int Hkv, int D, float scale, int window, float softcap, Tensor? gate) -> ()");
   m.def("value_mix(Tensor(a!) qkv, Tensor(b!) vfirst, Tensor? lam, int mix, int v_off, int v_cols) -> ()");
   m.def("gemm_any(Tensor(a!) out, Tensor x, Tensor w, Tensor? bias, int epi) -> ()");
   m.def("kv_store(Tensor qkv, Tensor(a!)? vfirst, Tensor? lam, int mix, Tensor(b!) kcache, Tensor(c!) vcache, Tensor tok_pos, Tensor tok_seq, Tensor block_table, int G, int d, int dv, int q_cols) -> ()");
@@ -924,6 +945,7 @@ TORCH_LIBRARY_IMPL(dlia, CUDA, m) {
   m.impl("gated_gelu", &gated_gelu);
   m.impl("paged_attention_window", &paged_attention_window);
   m.impl("paged_attention_biased", &paged_attention_biased);
+  m.impl("paged_attention_capped", &paged_attention_capped);
   m.impl("value_mix", &value_mix);
   m.impl("kv_store", &kv_store);
   m.impl("window_attention", &window_attention);

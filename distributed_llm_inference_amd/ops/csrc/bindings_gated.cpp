@@ -216,15 +216,22 @@ void moe_route(Tensor sel, Tensor wts, const Tensor& logits, int64_t top, int64_
                  cur_stream());
 }
 
-void moe_plan(Tensor tiles, Tensor row_tok, Tensor pair_row, const Tensor& sel, int64_t pairs, int64_t top, int64_t E, int64_t tile_rows) {
+void moe_plan(Tensor tiles, Tensor row_tok, Tensor pair_row, const Tensor& sel, int64_t pairs, int64_t top, int64_t E, int64_t tile_rows,
+              OptTensor wts, const std::optional<Tensor>& row_w) {
   DLIA_ON_DEVICE_OF(tiles);
   check_i32(tiles, "tiles"); check_i32(row_tok, "row_tok"); check_i32(pair_row, "pair_row"); check_i32(sel, "sel");
   DLIA_CHECK(tile_rows == 32 || tile_rows == 128, "moe: row tiles of 32 or 128");
   const int64_t max_tiles = (pairs + tile_rows - 1) / tile_rows + E;
   DLIA_CHECK(E >= 1 && E <= 256 && top >= 1 && pairs >= 0 && sel.numel() >= pairs && pair_row.numel() >= pairs, "moe_plan: pairs");
   DLIA_CHECK(tiles.numel() >= 1 + max_tiles && row_tok.numel() >= tile_rows * max_tiles, "moe_plan: room for pairs / tile_rows + E tiles");
+  float* rw = nullptr;
+  if (row_w.has_value()) {
+    check_f32(*row_w, "row_w");
+    DLIA_CHECK(row_w->numel() >= tile_rows * max_tiles && wts.has_value(), "moe_plan: row_w [rows] from the pairs' weights");
+    rw = row_w->data_ptr<float>();
+  }
   dlia_moe_plan(tiles.data_ptr<int>(), row_tok.data_ptr<int>(), pair_row.data_ptr<int>(), sel.data_ptr<int>(), (int)pairs, (int)top, (int)E,
-                (int)(tile_rows * max_tiles), (int)tile_rows, cur_stream());
+                (int)(tile_rows * max_tiles), (int)tile_rows, opt_f32(wts, pairs, "wts"), rw, cur_stream());
 }
 
 static void check_big(int64_t tile_rows, const Tensor& a, int64_t K, const Tensor& w) {
@@ -234,19 +241,27 @@ static void check_big(int64_t tile_rows, const Tensor& a, int64_t K, const Tenso
                reinterpret_cast<uintptr_t>(w.data_ptr()) % 16 == 0, "moe: 128-row tiles need bf16, K a multiple of 32 and 16-byte aligned rows");
 }
 
-void moe_up(Tensor act, const Tensor& x, const Tensor& wg, const Tensor& wu, const Tensor& tiles, const Tensor& row_tok, int64_t max_tiles,
-            double limit, int64_t tile_rows) {
+// Without wg the experts have no gate: act = relu(x . wu^T)^2. row_w [rows]: what the rows' inputs are multiplied by.
+void moe_up(Tensor act, const Tensor& x, OptTensor wg, const Tensor& wu, const Tensor& tiles, const Tensor& row_tok, int64_t max_tiles,
+            double limit, int64_t tile_rows, OptTensor row_w) {
   DLIA_ON_DEVICE_OF(act);
-  check_act(act, "act"); check_mat(act, "act"); check_act(x, "x"); check_mat(x, "x"); check_act(wg, "wg"); check_act(wu, "wu");
+  check_act(act, "act"); check_mat(act, "act"); check_act(x, "x"); check_mat(x, "x"); check_act(wu, "wu");
   check_i32(tiles, "tiles"); check_i32(row_tok, "row_tok");
-  DLIA_CHECK(wg.dim() == 3 && wg.is_contiguous() && wu.is_contiguous() && wu.sizes() == wg.sizes() && wg.size(2) == x.size(1) &&
-             x.scalar_type() == wg.scalar_type() && wu.scalar_type() == wg.scalar_type() && act.scalar_type() == x.scalar_type(),
-             "moe_up: x [T, K], wg / wu [E, F, K], one type");
-  check_big(tile_rows, x, x.size(1), wg);
-  DLIA_CHECK(act.size(1) == wg.size(1) && act.size(0) >= tile_rows * max_tiles && row_tok.numel() >= tile_rows * max_tiles && tiles.numel() >= 1 + max_tiles,
+  DLIA_CHECK(wu.dim() == 3 && wu.is_contiguous() && wu.size(2) == x.size(1) && wu.scalar_type() == x.scalar_type() && act.scalar_type() == x.scalar_type(),
+             "moe_up: x [T, K], wu [E, F, K], one type");
+  const void* gp = nullptr;
+  if (wg.has_value()) {
+    check_act(*wg, "wg");
+    DLIA_CHECK(wg->is_contiguous() && wu.sizes() == wg->sizes() && wg->scalar_type() == wu.scalar_type(), "moe_up: wg like wu");
+    check_big(tile_rows, x, x.size(1), *wg);
+    gp = wg->data_ptr();
+  }
+  check_big(tile_rows, x, x.size(1), wu);
+  DLIA_CHECK(act.size(1) == wu.size(1) && act.size(0) >= tile_rows * max_tiles && row_tok.numel() >= tile_rows * max_tiles && tiles.numel() >= 1 + max_tiles,
              "moe_up: act [tile_rows max_tiles, F]");
-  dlia_moe_up(act.data_ptr(), x.data_ptr(), wg.data_ptr(), wu.data_ptr(), is_f32(x), tiles.data_ptr<int>(), row_tok.data_ptr<int>(),
-              (int)max_tiles, x.size(0) > 256 ? 1 : 0, (int)wg.size(1), (int)wg.size(2), x.stride(0), act.stride(0), (float)limit, (int)tile_rows, cur_stream());
+  dlia_moe_up(act.data_ptr(), x.data_ptr(), gp, wu.data_ptr(), is_f32(x), tiles.data_ptr<int>(), row_tok.data_ptr<int>(),
+              (int)max_tiles, x.size(0) > 256 ? 1 : 0, (int)wu.size(1), (int)wu.size(2), x.stride(0), act.stride(0), (float)limit, (int)tile_rows,
+              opt_f32(row_w, tile_rows * max_tiles, "row_w"), cur_stream());
 }
 
 void moe_down(Tensor y, const Tensor& act, const Tensor& wd, const Tensor& tiles, const Tensor& row_tok, int64_t max_tiles, int64_t tile_rows) {
@@ -287,8 +302,8 @@ TORCH_LIBRARY_FRAGMENT(dlia, m) {
   m.def("state_scan_blocks(int d, int ncols) -> int");
   m.def("state_scan(int rule, Tensor(a!) o, Tensor z, Tensor? wz, Tensor(b!) state, Tensor(c!)? mstate, Tensor b0, Tensor? b1, Tensor q_start, Tensor ctx, Tensor slots, int H, int d, int dv, int col_q, int col_k, int col_v, int col_a, int col_i, int col_f, float cap, float qscale, int max_q, bool quick) -> ()");
   m.def("moe_route(Tensor(a!) sel, Tensor(b!) wts, Tensor logits, int top, int groups, int keep, float scale, Tensor? correction=None, bool softmax=False, int group_rank=2, bool renorm=True) -> ()");
-  m.def("moe_plan(Tensor(a!) tiles, Tensor(b!) row_tok, Tensor(c!) pair_row, Tensor sel, int pairs, int top, int E, int tile_rows) -> ()");
-  m.def("moe_up(Tensor(a!) act, Tensor x, Tensor wg, Tensor wu, Tensor tiles, Tensor row_tok, int max_tiles, float limit, int tile_rows) -> ()");
+  m.def("moe_plan(Tensor(a!) tiles, Tensor(b!) row_tok, Tensor(c!) pair_row, Tensor sel, int pairs, int top, int E, int tile_rows, Tensor? wts=None, Tensor(d!)? row_w=None) -> ()");
+  m.def("moe_up(Tensor(a!) act, Tensor x, Tensor? wg, Tensor wu, Tensor tiles, Tensor row_tok, int max_tiles, float limit, int tile_rows, Tensor? row_w=None) -> ()");
   m.def("moe_down(Tensor(a!) y, Tensor act, Tensor wd, Tensor tiles, Tensor row_tok, int max_tiles, int tile_rows) -> ()");
   m.def("moe_combine(Tensor(a!) out, Tensor y, Tensor pair_row, Tensor wts, int top, Tensor? x=None) -> ()");
 }

@@ -87,7 +87,9 @@ void dlia_paged_attention(void* out, const void* qkv, const void* kv_cache, cons
                           int Hkv, int D, int table_rows, int max_blocks, int num_blocks,
                           long ldq, long ldo, float scale, int splits, hipStream_t stream, int window = 0, int sink = 0,
                           const float* temp = nullptr, const float* bias = nullptr, int bias_rows = 0, const float* sinkv = nullptr,
-                          const float* gate = nullptr, long ldg = 0);
+                          const float* gate = nullptr, long ldg = 0, float softcap = 0.f, const void* egate = nullptr, long lde = 0);
+// (softcap > 0: scaled scores become cap tanh(score / cap); egate [T, lde] bf16: every entry of the output times the sigmoid of
+// its logit; with either of them neither sink nor the learned extras)
 // temp / bias / sinkv / gate (bf16 cache, sink set): a learned factor per head on the scores, a bias per (distance, head) and
 // the sink's score, both divided by `scale` by the caller, and a sigmoid gate logit per (token, head) on the head's output
 // (window > 0: a query at i sees the keys j with 0 <= i - j < window; sink: one more softmax term exp(0) without a value;
@@ -169,11 +171,13 @@ int dlia_state_scan(int rule, float* o, long ldo, const float* z, long ldz, cons
 // ---- moe.hip --------------------------------------------------------------------------------
 void dlia_moe_route(int* sel, float* wts, const float* logits, long ld, int T, int E, int top, int groups, int keep, float scale,
                     const float* corr, int softmax, int group_rank, int renorm, hipStream_t stream);
+// row_w (with wts): the pairs' weights at their rows
 void dlia_moe_plan(int* tiles, int* row_tok, int* pair_row, const int* sel, int pairs, int top, int E, int max_rows, int tile_rows,
-                   hipStream_t stream);
+                   const float* wts, float* row_w, hipStream_t stream);
 // tile_rows: 32 (register-tiled expert kernels, any type and shape) or 128 (LDS-tiled, bf16, K a multiple of 32, aligned rows)
+// wg null: experts without a gate, act = relu(x . Wu)^2; row_w: what the rows' inputs are multiplied by
 void dlia_moe_up(void* act, const void* x, const void* wg, const void* wu, int f32, const int* tiles, const int* row_tok,
-                 int max_tiles, int wide, int F, int K, long ldx, long lda, float limit, int tile_rows, hipStream_t stream);
+                 int max_tiles, int wide, int F, int K, long ldx, long lda, float limit, int tile_rows, const float* row_w, hipStream_t stream);
 void dlia_moe_down(float* y, const void* act, const void* wd, int f32, const int* tiles, const int* row_tok, int max_tiles, int wide,
                    int H, int F, long lda, int tile_rows, hipStream_t stream);
 // (wide: 128 / 256 output columns per workgroup, for steps with many rows; else 64)
@@ -261,6 +265,20 @@ long dlia_latent_attention_part_floats(int rows, int B, int H, int R);
 int dlia_latent_attention(void* out, const void* q, const void* kcache, const void* vt, const int* q_start, const int* ctx, const int* slots,
                           const int* block_table, int B, int T, int max_q, int max_blocks, int num_blocks, int table_rows, int H, int D,
                           int R, float scale, int window, float* part, long part_floats, hipStream_t stream);
+// ---- sandwich_ops.hip (plain-weight norms on both sides of every sublayer, bigram embedding, per-head q / k norms) ----
+void dlia_embed_bigram(float* out, void* cat, long ldc, int cat_both, const int* ids, const void* table, int f32, float scale, const void* bigram,
+                       int buckets, long mul_prev, long mul_cur, int* pages, const int* tok_pos, const int* tok_seq, const int* block_table,
+                       int T, int max_blocks, int num_blocks, int table_rows, int H, int vocab, hipStream_t stream);
+int dlia_sandwich_join_max_width(int vec);
+// Returns 1 (nothing launched) for rows wider than dlia_sandwich_join_max_width.
+int dlia_sandwich_join(void* out, int out_f32, long ldo, float* x, long ldx, const float* ya, long ldya, const float* yb, long ldyb, const float* ey,
+                       const int* pair_row, int top, const float* wb, const float* wn, int T, int H, float eps, hipStream_t stream);
+// Returns 1 (nothing launched) for types or sizes it does not take.
+int dlia_qk_prep(const void* z, int z_f32, long ldz, int T, int H, int G, int d, int dv, int col_v, const float* qw, const float* kw, int unit,
+                 float eps, int dims, int interleaved, const float* cos_t, const float* sin_t, int table_pos, void* q_out, int q_f32, long ldqo,
+                 void* kc, void* vc, int cache_f32, int layout, const int* tok_pos, const int* tok_seq, const int* block_table, int max_blocks,
+                 int num_blocks, int table_rows, hipStream_t stream);
+void dlia_relu_act(void* act, int out_f32, long lda, const void* z, int z_f32, long ldz, int M, int F, int glu, hipStream_t stream);
 // ---- misc.hip -------------------------------------------------------------------------
 void dlia_advance_i32(int* x, int n, int delta, hipStream_t stream);
 void dlia_scatter_rows_i32(int* dst, const int* rows, const int* src, int nrows, int ncols, int dst_rows, hipStream_t stream);

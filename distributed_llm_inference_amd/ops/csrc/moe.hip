@@ -19,7 +19,8 @@
 //                multiplies the row) in fp32
 //   moe_up       grid (column blocks, tiles): act[row, f] = g s(1.702 g) (u + 1), g = min(x . Wg[e][f], limit),
 //                u = clamp(x . Wu[e][f], -limit, limit), x the row's token; with limit <= 0 the plain silu(g) * u.
-//                Gate and up accumulate over the same A fragments.
+//                Gate and up accumulate over the same A fragments. Experts without a gate: act = relu(x . Wu[e][f])^2. With
+//                weights per row (the plan lays them out) x is the token times its weight: the products are multiplied by it.
 //   moe_down     y[row, c] = act[row] . Wd[e][c] in fp32.
 //   moe_combine  out[t, :] = sum over the token's choices of weight * y[row, :], in the order of the choices (fp32); a choice
 //                without a row (an identity expert) contributes weight * x[t, :].
@@ -42,6 +43,8 @@ __device__ __forceinline__ float expert_act(float g, float u, float limit) {
   }
   return g / (1.f + expf(-g)) * u;
 }
+
+__device__ __forceinline__ float relu2(float u) { const float r = fmaxf(u, 0.f); return r * r; }
 
 __global__ __launch_bounds__(64) void moe_route_kernel(int* __restrict__ sel, float* __restrict__ wts,
                                                        const float* __restrict__ logits, long ld, int T, int E, int top,
@@ -103,7 +106,7 @@ __global__ __launch_bounds__(64) void moe_route_kernel(int* __restrict__ sel, fl
 template <typename Sel>
 __device__ __forceinline__ void plan_pairs(int* __restrict__ tiles, int* __restrict__ row_tok, int* __restrict__ pair_row, int pairs,
                                            int top, int E, int max_rows, int tile_rows, int* count, int* start, int* fill, int* ntiles,
-                                           Sel expert) {
+                                           Sel expert, const float* __restrict__ wts = nullptr, float* __restrict__ row_w = nullptr) {
   for (int e = threadIdx.x; e < E; e += 1024) { count[e] = 0; fill[e] = 0; }
   __syncthreads();
   for (int i = threadIdx.x; i < pairs; i += 1024) {
@@ -130,16 +133,17 @@ __device__ __forceinline__ void plan_pairs(int* __restrict__ tiles, int* __restr
     const int e = expert(i);
     if (e >= E) { pair_row[i] = -1; continue; }                      // (an identity expert: no row)
     const int r = start[e] + atomicAdd(&fill[e], 1);
-    if (r < max_rows && r < used) { row_tok[r] = i / top; pair_row[i] = r; }
+    if (r < max_rows && r < used) { row_tok[r] = i / top; pair_row[i] = r; if (row_w) row_w[r] = wts[i]; }
   }
 }
 
 __global__ __launch_bounds__(1024) void moe_plan_kernel(int* __restrict__ tiles, int* __restrict__ row_tok,
                                                         int* __restrict__ pair_row, const int* __restrict__ sel, int pairs,
-                                                        int top, int E, int max_rows, int tile_rows) {
+                                                        int top, int E, int max_rows, int tile_rows, const float* __restrict__ wts,
+                                                        float* __restrict__ row_w) {
   __shared__ int count[kMoeMaxExperts], start[kMoeMaxExperts], fill[kMoeMaxExperts];
   __shared__ int ntiles;
-  plan_pairs(tiles, row_tok, pair_row, pairs, top, E, max_rows, tile_rows, count, start, fill, &ntiles, [&](int i) { return sel[i]; });
+  plan_pairs(tiles, row_tok, pair_row, pairs, top, E, max_rows, tile_rows, count, start, fill, &ntiles, [&](int i) { return sel[i]; }, wts, row_w);
 }
 
 constexpr int kPlanDesc = 8;
@@ -181,11 +185,11 @@ __global__ __launch_bounds__(256) void glu_act_kernel(OT* __restrict__ act, long
 // and the fragments of the next k-step are on their way while the current ones are multiplied.
 constexpr int kMoeTile = kMoeRows;
 
-template <typename T, typename OT, int NJ>
+template <typename T, typename OT, int NJ, bool GLU>
 __global__ __launch_bounds__(256) void moe_up_kernel(OT* __restrict__ act, const T* __restrict__ x, const T* __restrict__ wg,
                                                      const T* __restrict__ wu, const int* __restrict__ tiles,
                                                      const int* __restrict__ row_tok, int F, int K, long ldx, long lda,
-                                                     float limit, int vec_ok) {
+                                                     float limit, int vec_ok, const float* __restrict__ row_w) {
   constexpr int VEC = 16 / sizeof(T), KS = 4 * VEC;
   const int tile = blockIdx.y;
   if (tile >= tiles[0]) return;
@@ -217,7 +221,7 @@ __global__ __launch_bounds__(256) void moe_up_kernel(OT* __restrict__ act, const
     for (int i = 0; i < 2; ++i) fa[i] = load_frag<T>(arow[i], k, K, av[i], vec_ok);
 #pragma unroll
     for (int j = 0; j < NJ; ++j) {
-      fg[j] = load_frag<T>(wg + wrow[j], k, K, wv[j], vec_ok);
+      if constexpr (GLU) fg[j] = load_frag<T>(wg + wrow[j], k, K, wv[j], vec_ok);
       fu[j] = load_frag<T>(wu + wrow[j], k, K, wv[j], vec_ok);
     }
   };
@@ -227,11 +231,14 @@ __global__ __launch_bounds__(256) void moe_up_kernel(OT* __restrict__ act, const
 #pragma unroll
     for (int i = 0; i < 2; ++i)
 #pragma unroll
-      for (int j = 0; j < NJ; ++j) { ag[i][j] = mma_frag(T{}, a[i], g[j], ag[i][j]); au[i][j] = mma_frag(T{}, a[i], u[j], au[i][j]); }
+      for (int j = 0; j < NJ; ++j) {
+        if constexpr (GLU) ag[i][j] = mma_frag(T{}, a[i], g[j], ag[i][j]);
+        au[i][j] = mma_frag(T{}, a[i], u[j], au[i][j]);
+      }
 #pragma unroll
     for (int i = 0; i < 2; ++i) a[i] = an[i];
 #pragma unroll
-    for (int j = 0; j < NJ; ++j) { g[j] = gn[j]; u[j] = un[j]; }
+    for (int j = 0; j < NJ; ++j) { if constexpr (GLU) g[j] = gn[j]; u[j] = un[j]; }
   }
 #pragma unroll
   for (int i = 0; i < 2; ++i)
@@ -242,7 +249,9 @@ __global__ __launch_bounds__(256) void moe_up_kernel(OT* __restrict__ act, const
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
         const int row = tile * kMoeTile + i * 16 + kq * 4 + r;
-        act[(long)row * lda + col] = (OT)expert_act(ag[i][j][r], au[i][j][r], limit);
+        const float rw = row_w && row_tok[row] >= 0 ? row_w[row] : 1.f;      // (padding rows have no weight)
+        if constexpr (GLU) act[(long)row * lda + col] = (OT)expert_act(ag[i][j][r] * rw, au[i][j][r] * rw, limit);
+        else act[(long)row * lda + col] = (OT)relu2(au[i][j][r] * rw);
       }
     }
 }
@@ -314,17 +323,19 @@ __global__ __launch_bounds__(256) void moe_down_kernel(float* __restrict__ y, co
 // MFMAs. bf16, K a multiple of 32 with 16-byte aligned rows (the caller falls back to the register-tiled kernels otherwise).
 constexpr int kBigStride = 40;          // bf16 elements between rows in LDS (64 bytes of data + 16 of padding)
 
-template <bool UP>
+// KIND 0: down; 1: gate and up; 2: up alone (128 columns per workgroup, the square of relu).
+template <int KIND>
 __global__ __launch_bounds__(256) void moe_big_kernel(bf16* __restrict__ act_out, float* __restrict__ y_out, const bf16* __restrict__ a,
                                                       const bf16* __restrict__ w0, const bf16* __restrict__ w1,
                                                       const int* __restrict__ tiles, const int* __restrict__ row_tok, int N, int K,
-                                                      long lda, long ldo, float limit) {
+                                                      long lda, long ldo, float limit, const float* __restrict__ row_w) {
+  constexpr bool UP = KIND >= 1, GLU = KIND == 1;
   __shared__ __attribute__((aligned(16))) bf16 lds[2][256 * kBigStride];
   const int tile = blockIdx.y;
   if (tile >= tiles[0]) return;
   const int e = tiles[1 + tile];
   const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, r16 = lane & 15, kq = lane >> 4;
-  const int n0 = blockIdx.x * (UP ? 64 : 128);                  // first output column of the workgroup
+  const int n0 = blockIdx.x * (GLU ? 64 : 128);                 // first output column of the workgroup
   // the four pieces this thread stages per k-step: pieces 2 tid, 2 tid + 1 of the 512 row pieces, and of the 512 weight pieces
   const bf16* src[4]; bool ok[4]; int dst[4];
 #pragma unroll
@@ -336,7 +347,7 @@ __global__ __launch_bounds__(256) void moe_big_kernel(bf16* __restrict__ act_out
     dst[i] = row * kBigStride + part * 8;
     // weights: LDS rows 128 .. 255
     int wr; const bf16* base;
-    if constexpr (UP) { wr = n0 + (row & 63); base = row < 64 ? w0 : w1; }
+    if constexpr (GLU) { wr = n0 + (row & 63); base = row < 64 ? w0 : w1; }
     else { wr = n0 + row; base = w0; }
     ok[2 + i] = wr < N;
     src[2 + i] = base + ((long)e * N + (ok[2 + i] ? wr : 0)) * K + part * 8;
@@ -381,12 +392,20 @@ __global__ __launch_bounds__(256) void moe_big_kernel(bf16* __restrict__ act_out
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
       const long row = (long)tile * kMoeBigRows + wave * 32 + i * 16 + kq * 4 + r;
-      if constexpr (UP) {
+      [[maybe_unused]] float rw = 1.f;
+      if constexpr (UP) { if (row_w && row_tok[row] >= 0) rw = row_w[row]; }
+      if constexpr (GLU) {
 #pragma unroll
         for (int j = 0; j < 4; ++j) {
           const int col = n0 + j * 16 + r16;
           if (col >= N) continue;
-          act_out[row * ldo + col] = (bf16)expert_act(acc[i][j][r], acc[i][j + 4][r], limit);
+          act_out[row * ldo + col] = (bf16)expert_act(acc[i][j][r] * rw, acc[i][j + 4][r] * rw, limit);
+        }
+      } else if constexpr (UP) {
+#pragma unroll
+        for (int j = 0; j < 8; ++j) {
+          const int col = n0 + j * 16 + r16;
+          if (col < N) act_out[row * ldo + col] = (bf16)relu2(acc[i][j][r] * rw);
         }
       } else {
 #pragma unroll
@@ -422,18 +441,22 @@ extern "C" void dlia_moe_route(int* sel, float* wts, const float* logits, long l
 }
 
 extern "C" void dlia_moe_plan(int* tiles, int* row_tok, int* pair_row, const int* sel, int pairs, int top, int E, int max_rows,
-                              int tile_rows, hipStream_t stream) {
+                              int tile_rows, const float* wts, float* row_w, hipStream_t stream) {
   hipLaunchKernelGGL(dlia::moe_plan_kernel, dim3(1), dim3(1024), 0, stream, tiles, row_tok, pair_row, sel, pairs, top, E, max_rows,
-                     tile_rows);
+                     tile_rows, wts, row_w);
 }
 
 // Steps with few rows (decoding) take narrow column blocks: more workgroups stream the experts' weights at once.
 template <typename T, typename OT, int NJ>
 static void launch_moe_up(void* act, const void* x, const void* wg, const void* wu, const int* tiles, const int* row_tok, int max_tiles,
-                          int F, int K, long ldx, long lda, float limit, int ok, hipStream_t stream) {
+                          int F, int K, long ldx, long lda, float limit, int ok, const float* row_w, hipStream_t stream) {
   const dim3 grid((F + 64 * NJ - 1) / (64 * NJ), max_tiles);
-  hipLaunchKernelGGL((dlia::moe_up_kernel<T, OT, NJ>), grid, dim3(256), 0, stream, (OT*)act, (const T*)x, (const T*)wg, (const T*)wu,
-                     tiles, row_tok, F, K, ldx, lda, limit, ok);
+  if (wg)
+    hipLaunchKernelGGL((dlia::moe_up_kernel<T, OT, NJ, true>), grid, dim3(256), 0, stream, (OT*)act, (const T*)x, (const T*)wg, (const T*)wu,
+                       tiles, row_tok, F, K, ldx, lda, limit, ok, row_w);
+  else
+    hipLaunchKernelGGL((dlia::moe_up_kernel<T, OT, NJ, false>), grid, dim3(256), 0, stream, (OT*)act, (const T*)x, (const T*)wg, (const T*)wu,
+                       tiles, row_tok, F, K, ldx, lda, limit, ok, row_w);
 }
 template <typename T, int NJ>
 static void launch_moe_down(float* y, const void* act, const void* wd, const int* tiles, const int* row_tok, int max_tiles, int H, int F,
@@ -443,21 +466,26 @@ static void launch_moe_down(float* y, const void* act, const void* wd, const int
 }
 
 extern "C" void dlia_moe_up(void* act, const void* x, const void* wg, const void* wu, int f32, const int* tiles, const int* row_tok,
-                            int max_tiles, int wide, int F, int K, long ldx, long lda, float limit, int tile_rows, hipStream_t stream) {
+                            int max_tiles, int wide, int F, int K, long ldx, long lda, float limit, int tile_rows, const float* row_w,
+                            hipStream_t stream) {
   if (max_tiles <= 0) return;
   if (tile_rows == dlia::kMoeBigRows) {
-    hipLaunchKernelGGL(dlia::moe_big_kernel<true>, dim3((F + 63) / 64, max_tiles), dim3(256), 0, stream, (dlia::bf16*)act, (float*)nullptr,
-                       (const dlia::bf16*)x, (const dlia::bf16*)wg, (const dlia::bf16*)wu, tiles, row_tok, F, K, ldx, lda, limit);
+    if (wg)
+      hipLaunchKernelGGL(dlia::moe_big_kernel<1>, dim3((F + 63) / 64, max_tiles), dim3(256), 0, stream, (dlia::bf16*)act, (float*)nullptr,
+                         (const dlia::bf16*)x, (const dlia::bf16*)wg, (const dlia::bf16*)wu, tiles, row_tok, F, K, ldx, lda, limit, row_w);
+    else
+      hipLaunchKernelGGL(dlia::moe_big_kernel<2>, dim3((F + 127) / 128, max_tiles), dim3(256), 0, stream, (dlia::bf16*)act, (float*)nullptr,
+                         (const dlia::bf16*)x, (const dlia::bf16*)wu, (const dlia::bf16*)nullptr, tiles, row_tok, F, K, ldx, lda, limit, row_w);
     return;
   }
   const int vec = f32 ? 4 : 8;
   const int ok = K % vec == 0 && ldx % vec == 0 && (uintptr_t)x % 16 == 0 && (uintptr_t)wg % 16 == 0 && (uintptr_t)wu % 16 == 0;
   if (f32) {
-    if (wide) launch_moe_up<float, float, 2>(act, x, wg, wu, tiles, row_tok, max_tiles, F, K, ldx, lda, limit, ok, stream);
-    else launch_moe_up<float, float, 1>(act, x, wg, wu, tiles, row_tok, max_tiles, F, K, ldx, lda, limit, ok, stream);
+    if (wide) launch_moe_up<float, float, 2>(act, x, wg, wu, tiles, row_tok, max_tiles, F, K, ldx, lda, limit, ok, row_w, stream);
+    else launch_moe_up<float, float, 1>(act, x, wg, wu, tiles, row_tok, max_tiles, F, K, ldx, lda, limit, ok, row_w, stream);
   } else {
-    if (wide) launch_moe_up<dlia::bf16, dlia::bf16, 2>(act, x, wg, wu, tiles, row_tok, max_tiles, F, K, ldx, lda, limit, ok, stream);
-    else launch_moe_up<dlia::bf16, dlia::bf16, 1>(act, x, wg, wu, tiles, row_tok, max_tiles, F, K, ldx, lda, limit, ok, stream);
+    if (wide) launch_moe_up<dlia::bf16, dlia::bf16, 2>(act, x, wg, wu, tiles, row_tok, max_tiles, F, K, ldx, lda, limit, ok, row_w, stream);
+    else launch_moe_up<dlia::bf16, dlia::bf16, 1>(act, x, wg, wu, tiles, row_tok, max_tiles, F, K, ldx, lda, limit, ok, row_w, stream);
   }
 }
 
@@ -465,8 +493,9 @@ extern "C" void dlia_moe_down(float* y, const void* act, const void* wd, int f32
                               int max_tiles, int wide, int H, int F, long lda, int tile_rows, hipStream_t stream) {
   if (max_tiles <= 0) return;
   if (tile_rows == dlia::kMoeBigRows) {
-    hipLaunchKernelGGL(dlia::moe_big_kernel<false>, dim3((H + 127) / 128, max_tiles), dim3(256), 0, stream, (dlia::bf16*)nullptr, y,
-                       (const dlia::bf16*)act, (const dlia::bf16*)wd, (const dlia::bf16*)nullptr, tiles, row_tok, H, F, lda, (long)H, 0.f);
+    hipLaunchKernelGGL(dlia::moe_big_kernel<0>, dim3((H + 127) / 128, max_tiles), dim3(256), 0, stream, (dlia::bf16*)nullptr, y,
+                       (const dlia::bf16*)act, (const dlia::bf16*)wd, (const dlia::bf16*)nullptr, tiles, row_tok, H, F, lda, (long)H, 0.f,
+                       (const float*)nullptr);
     return;
   }
   const int vec = f32 ? 4 : 8;
