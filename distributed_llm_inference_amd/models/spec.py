@@ -741,7 +741,7 @@ class ModelSpec:
                 raise ValueError(f"layer {i}: {rd} rotated entries of {d}")
             win = (m.get("mask") or {}).get("size")
             common = dict(heads=H, kv_heads=G, dim=d, vdim=dv, scale=float(m.get("scale", d ** -0.5)), window=int(win) if win else None,
-                          softcap=float(m.get("softcap") or 0.0), rope_dims=rd, rope_base=float(rot.get("base", 10000.0)), **ffkw)
+                          softcap=float(m.get("softcap") or 0.0), rope_dims=rd, rope_base=float(rot["base"]) if rd else 10000.0, **ffkw)
             if l["type"] == "attention":
                 layers.append(LayerSpec("attention", head_norm=True, **common))
             elif l["type"] == "attention_2":
