@@ -2,7 +2,8 @@
 Nufapel stack beside the Letarax stack of equal size (`bench.py --gated-compare`), of a Tezesun stack beside the
 Letarax stack of equal size (`bench.py --parallel-compare`), of a Zovozen stack beside the Nufapel stack of equal size
 (`bench.py --postnorm-compare`), and of a Pifutar stack beside the Nufapel and the Tezesun stack of equal size
-(`bench.py --canon-compare`).
+(`bench.py --canon-compare`), and of a Migenex stack beside the Letarax and the Nufapel stack of equal size
+(`bench.py --sandwich-compare`).
 
 Both models get random weights and the same width, head counts, head size, feed-forward width, depth and
 vocabulary; the Letarax stack has three attention layers (windowed, with the sink and value mixing) to one delta-rule
@@ -53,6 +54,15 @@ def canon_specs(name: str):
     mechanisms: Nufapel (matrix states in the slots, routed feed-forwards) and Tezesun (latent attention, dense feed-forwards)."""
     from distributed_llm_inference_amd.models.spec import BUILTIN_SPECS
     return tuple(BUILTIN_SPECS[f"{f}-{name}"] for f in ("pifutar", "nufapel", "tezesun"))
+
+
+def sandwich_specs(name: str):
+    """The Migenex stack of a size (three windowed layers whose keys are their values to one over the whole context with capped scores;
+    dense and routed feed-forwards alternating; one pass behind the map) beside the two existing designs that share its mechanisms:
+    Letarax (norms on both sides of every sublayer, windowed attention, dense gated feed-forwards) and Nufapel (a repeated stretch,
+    attention over the whole context, routed feed-forwards)."""
+    from distributed_llm_inference_amd.models.spec import BUILTIN_SPECS
+    return tuple(BUILTIN_SPECS[f"{f}-{name}"] for f in ("migenex", "letarax", "nufapel"))
 
 
 def specs(name: str):
@@ -120,12 +130,12 @@ def time_decode(ex, rows: int, ctx: int, iters: int) -> float:
 
 
 def main(sizes=None, iters: int = 8, out=sys.stdout, gated: bool = False, parallel: bool = False, postnorm: bool = False,
-         canon: bool = False) -> int:
+         canon: bool = False, sandwich: bool = False) -> int:
     import gc
     import torch
     rows, ctx, plen = 64, 1024, 2048
     for name in (sizes or list(SIZES)):
-        pair = canon_specs(name) if canon else postnorm_specs(name) if postnorm else parallel_specs(name) if parallel else gated_specs(name) if gated else specs(name)
+        pair = sandwich_specs(name) if sandwich else canon_specs(name) if canon else postnorm_specs(name) if postnorm else parallel_specs(name) if parallel else gated_specs(name) if gated else specs(name)
         new, *old = [x.family for x in pair]
         rec = {"metric": f"{new}_vs_{'_'.join(old)}_tokens_per_s", "size": name, "dtype": "bf16", "data": "synthetic", "weights": "random",
                "config": dict(zip(("width", "heads", "kv_heads", "head_dim", "ff", "layers", "window"), SIZES[name])),
