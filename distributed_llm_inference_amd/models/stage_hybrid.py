@@ -164,6 +164,7 @@ class HybridGpuStage(GpuStage):
         self.decode_rows = 256
         # latent attention in bf16: DLIA_LATENT_ATTN=0 keeps it on the general tile kernel (A/B)
         self._latent_fast = os.environ.get("DLIA_LATENT_ATTN", "1") != "0"
+        self._part_cfg: Dict[tuple, tuple] = {}
         self._shapes = []                        # (N, K, has_bias) of every packed GEMM, for the workspace
         # Attention layers whose keys and values have one size, 64 or 128, with up to 16 query heads per key / value head run
         # on the library's MFMA attention kernels (fragment-ordered cache, the windowed / sink instantiations), bf16 only;
@@ -351,6 +352,21 @@ class HybridGpuStage(GpuStage):
         # more than 256 rows: the tile kernel, spread over the whole chip when a shape has few tiles
         self.K.gemm(out, x, wp, b, None, wk.ws, p[name + "_n"], 1 if b is not None else 0, 256 if x.shape[0] > self.decode_rows else 0, 0)
 
+    def _mm_parts(self, wk, out: torch.Tensor, x: torch.Tensor, p, name: str, cols: int) -> torch.Tensor:
+        """x . W^T for a consumer that adds up the partial results of key splits while it reads them: [splits, T, cols] in the step's
+        GEMM workspace for steps on the weight-streaming kernel (valid until the next GEMM), else [T, cols] in `out`."""
+        T, wp = x.shape[0], p.get(name + "_p")
+        if wp is None or T > self.decode_rows:
+            self._mm(wk, out, x, p, name)
+            return out[:, :cols]
+        n4 = p[name + "_n"]
+        key = (T, n4, x.shape[1])
+        cfg = self._part_cfg.get(key)
+        if cfg is None:
+            cfg = self._part_cfg[key] = tuple(int(v) for v in self.K.gemm_config(T, n4, x.shape[1], 6, True))
+        self.K.gemm(out, x, wp, None, None, wk.ws, n4, 6, cfg[1], cfg[0])
+        return wk.ws[:cfg[1] * T * n4].view(cfg[1], T, n4)[:, :, :cols]
+
     def _packed_ws_floats(self) -> int:
         need = 1
         for (n_, k_, hb) in self._shapes:
@@ -358,6 +374,8 @@ class HybridGpuStage(GpuStage):
                 sk = int(self.K.gemm_config(m_, n_, k_, 1 if hb else 0, True)[1])
                 if sk > 1:
                     need = max(need, sk * m_ * n_)
+                if self.sand:                # (partial results that the next kernel adds up, `_mm_parts`)
+                    need = max(need, int(self.K.gemm_config(m_, n_, k_, 6, True)[1]) * m_ * n_)
         return need
 
     # ---- workspaces ---------------------------------------------------------------------------------------
@@ -1502,20 +1520,20 @@ class HybridGpuStage(GpuStage):
         def enter(ri):
             """The stream, in the map's input type, becomes the pass's first stream; its norm is what run ri reads."""
             self._mm(wk, h, wk.cat[:T], self.loop_p, "w_loop")
-            K.sandwich_join(xn, h, None, None, None, None, 1, None, self.layers[runs[ri][0]]["ln1_w"], eps)
+            K.sandwich_join(xn, h, None, None, None, 1, None, self.layers[runs[ri][0]]["ln1_w"], eps)
 
-        def join(wb, wn, follows, ya=None, yb=None, ey=None, top=1):
+        def join(wb, wn, follows, ya=None, ey=None, top=1):
             """Adds a sublayer's output; `wn`: the norm of the sublayer that reads next, else the run `follows` does."""
             out = xn
             if wn is None and follows is not None:
                 out = None if follows >= len(runs) else wk.cat[:T, :H] if opens(follows) else xn
                 wn = self.layers[runs[follows][0]]["ln1_w"] if out is xn else None
-            K.sandwich_join(out, h, ya, yb, ey, wk.pair_row if ey is not None else None, top, wb, wn, eps)
+            K.sandwich_join(out, h, ya, ey, wk.pair_row if ey is not None else None, top, wb, wn, eps)
 
         if opens(0):
             enter(0)             # (the embedding left the stream in both halves of the map's input)
         else:
-            K.sandwich_join(xn, h, None, None, None, None, 1, None, self.layers[runs[0][0]]["ln1_w"], eps)
+            K.sandwich_join(xn, h, None, None, None, 1, None, self.layers[runs[0][0]]["ln1_w"], eps)
         for ri, (li, _) in enumerate(runs):
             ls, p = self.specs[li], self.layers[li]
             Hh, G, d, dv, fast, tile = ls.heads, ls.kv_heads, ls.dim, ls.vdim, self.mfma_attn[ri], self._tile[ri]
@@ -1540,9 +1558,8 @@ class HybridGpuStage(GpuStage):
                                      win, 0, ls.softcap, 0.0, 1.0, eps, gate[:r1] if gate is not None else None, wk.part)
                 else:
                     K.multi_attention(mixed, q, d, kc, vc, 0, tok_pos, tok_seq, table, Hh, d, dv, 1, ls.scale, win, 0, ls.softcap, 0.0, 1.0, eps, gate)
-            ya = view(wk.ya, self._cols(p, "w_o"))
-            self._mm(wk, ya, mixed, p, "w_o")
-            join(p["ln1b_w"], p["ln2_w"] if ls.has_ff else None, ri + 1, ya[:, :H])
+            ya = self._mm_parts(wk, view(wk.ya, self._cols(p, "w_o")), mixed, p, "w_o", H)
+            join(p["ln1b_w"], p["ln2_w"] if ls.has_ff else None, ri + 1, ya)
             if ls.moe is not None:
                 e = ls.moe
                 z2 = view(wk.z2, self._cols(p, "w_ff"))
@@ -1552,23 +1569,21 @@ class HybridGpuStage(GpuStage):
                 tr = 128 if (self.wmode == "bf16" and T * e.top >= 1024 and H % 32 == 0 and e.ff % 32 == 0) else 32
                 nt = (T * e.top + tr - 1) // tr + e.experts
                 eact, ey = wk.eact[:tr * nt * e.ff].view(tr * nt, e.ff), wk.ey[:tr * nt * H].view(tr * nt, H)
-                K.moe_route(wk.sel, wk.wts, z2[:, :e.outputs], e.top, e.groups, e.keep, e.scale, None, e.score == "softmax", e.group_rank, e.renorm)
-                K.moe_plan(wk.tiles, wk.row_tok, wk.pair_row, wk.sel, T * e.top, e.top, e.experts, tr, wk.wts, wk.row_w)
+                K.moe_route_plan(wk.sel, wk.wts, z2[:, :e.outputs], e.top, e.groups, e.keep, e.scale, None, e.score == "softmax", e.group_rank, e.renorm,
+                                 wk.tiles, wk.row_tok, wk.pair_row, e.experts, tr, wk.row_w)
                 K.moe_up(eact, xn, None, p["w_up_e"], wk.tiles, wk.row_tok, nt, 0.0, tr, wk.row_w)
                 K.moe_down(ey, eact, p["w_down_e"], wk.tiles, wk.row_tok, nt, tr)
-                yb = None
+                ya = None
                 if e.shared_ff:
-                    act, yb = view(wk.act, e.shared_ff), view(wk.ya, self._cols(p, "w_down_s"))
+                    act = view(wk.act, e.shared_ff)
                     K.relu_act(act, z2[:, e.outputs:e.outputs + e.shared_ff], False)
-                    self._mm(wk, yb, act, p, "w_down_s")
-                    yb = yb[:, :H]
-                join(p["ln2b_w"], None, ri + 1, None, yb, ey, e.top)
+                    ya = self._mm_parts(wk, view(wk.ya, self._cols(p, "w_down_s")), act, p, "w_down_s", H)
+                join(p["ln2b_w"], None, ri + 1, ya, ey, e.top)
             elif ls.ff:
-                gu, act, ya = view(wk.gu, self._cols(p, "w_gu")), view(wk.act, ls.ff), view(wk.ya, self._cols(p, "w_down"))
+                gu, act = view(wk.gu, self._cols(p, "w_gu")), view(wk.act, ls.ff)
                 self._mm(wk, gu, xn, p, "w_gu")
                 K.relu_act(act, gu, True)
-                self._mm(wk, ya, act, p, "w_down")
-                join(p["ln2b_w"], None, ri + 1, ya[:, :H])
+                join(p["ln2b_w"], None, ri + 1, self._mm_parts(wk, view(wk.ya, self._cols(p, "w_down")), act, p, "w_down", H))
             if keep:
                 self.layer_outputs.append(h.clone())
             if opens(ri + 1):

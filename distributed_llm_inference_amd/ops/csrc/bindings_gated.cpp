@@ -234,6 +234,32 @@ void moe_plan(Tensor tiles, Tensor row_tok, Tensor pair_row, const Tensor& sel, 
                 (int)(tile_rows * max_tiles), (int)tile_rows, opt_f32(wts, pairs, "wts"), rw, cur_stream());
 }
 
+// moe_route, then moe_plan over its choices (E: the experts that have rows)
+void moe_route_plan(Tensor sel, Tensor wts, const Tensor& logits, int64_t top, int64_t groups, int64_t keep, double scale, OptTensor correction,
+                    bool softmax, int64_t group_rank, bool renorm, Tensor tiles, Tensor row_tok, Tensor pair_row, int64_t E, int64_t tile_rows,
+                    const std::optional<Tensor>& row_w) {
+  DLIA_ON_DEVICE_OF(sel);
+  check_i32(sel, "sel"); check_f32(wts, "wts"); check_fmat(logits, "logits");
+  check_i32(tiles, "tiles"); check_i32(row_tok, "row_tok"); check_i32(pair_row, "pair_row");
+  const int64_t T = logits.size(0), outs = logits.size(1), pairs = T * top;
+  DLIA_CHECK(outs >= 1 && outs <= 256 && E >= 1 && E <= outs && groups >= 1 && outs % groups == 0 && keep >= 1 && keep <= groups && top >= 1 &&
+             top <= keep * (outs / groups), "moe_route_plan: up to 256 experts in equal groups, top within the kept groups");
+  DLIA_CHECK(sel.numel() >= pairs && wts.numel() >= pairs && pair_row.numel() >= pairs && (group_rank == 1 || group_rank == 2) &&
+             (tile_rows == 32 || tile_rows == 128), "moe_route_plan: sel / wts / pair_row [T, top], row tiles of 32 or 128");
+  const int64_t max_tiles = (pairs + tile_rows - 1) / tile_rows + E;
+  DLIA_CHECK(tiles.numel() >= 1 + max_tiles && row_tok.numel() >= tile_rows * max_tiles, "moe_route_plan: room for pairs / tile_rows + E tiles");
+  float* rw = nullptr;
+  if (row_w.has_value()) {
+    check_f32(*row_w, "row_w");
+    DLIA_CHECK(row_w->numel() >= tile_rows * max_tiles, "moe_route_plan: row_w [rows]");
+    rw = row_w->data_ptr<float>();
+  }
+  dlia_moe_route_plan(sel.data_ptr<int>(), wts.data_ptr<float>(), logits.data_ptr<float>(), logits.stride(0), (int)T, (int)outs, (int)top, (int)groups,
+                      (int)keep, (float)scale, opt_f32(correction, outs, "correction"), softmax ? 1 : 0, (int)group_rank, renorm ? 1 : 0,
+                      tiles.data_ptr<int>(), row_tok.data_ptr<int>(), pair_row.data_ptr<int>(), (int)E, (int)(tile_rows * max_tiles), (int)tile_rows,
+                      rw, cur_stream());
+}
+
 static void check_big(int64_t tile_rows, const Tensor& a, int64_t K, const Tensor& w) {
   DLIA_CHECK(tile_rows == 32 || tile_rows == 128, "moe: row tiles of 32 or 128");
   if (tile_rows == 128)
@@ -303,6 +329,7 @@ TORCH_LIBRARY_FRAGMENT(dlia, m) {
   m.def("state_scan(int rule, Tensor(a!) o, Tensor z, Tensor? wz, Tensor(b!) state, Tensor(c!)? mstate, Tensor b0, Tensor? b1, Tensor q_start, Tensor ctx, Tensor slots, int H, int d, int dv, int col_q, int col_k, int col_v, int col_a, int col_i, int col_f, float cap, float qscale, int max_q, bool quick) -> ()");
   m.def("moe_route(Tensor(a!) sel, Tensor(b!) wts, Tensor logits, int top, int groups, int keep, float scale, Tensor? correction=None, bool softmax=False, int group_rank=2, bool renorm=True) -> ()");
   m.def("moe_plan(Tensor(a!) tiles, Tensor(b!) row_tok, Tensor(c!) pair_row, Tensor sel, int pairs, int top, int E, int tile_rows, Tensor? wts=None, Tensor(d!)? row_w=None) -> ()");
+  m.def("moe_route_plan(Tensor(a!) sel, Tensor(b!) wts, Tensor logits, int top, int groups, int keep, float scale, Tensor? correction, bool softmax, int group_rank, bool renorm, Tensor(c!) tiles, Tensor(d!) row_tok, Tensor(e!) pair_row, int E, int tile_rows, Tensor(f!)? row_w) -> ()");
   m.def("moe_up(Tensor(a!) act, Tensor x, Tensor? wg, Tensor wu, Tensor tiles, Tensor row_tok, int max_tiles, float limit, int tile_rows, Tensor? row_w=None) -> ()");
   m.def("moe_down(Tensor(a!) y, Tensor act, Tensor wd, Tensor tiles, Tensor row_tok, int max_tiles, int tile_rows) -> ()");
   m.def("moe_combine(Tensor(a!) out, Tensor y, Tensor pair_row, Tensor wts, int top, Tensor? x=None) -> ()");
@@ -318,6 +345,7 @@ TORCH_LIBRARY_IMPL(dlia, CUDA, m) {
   m.impl("state_scan", &state_scan);
   m.impl("moe_route", &moe_route);
   m.impl("moe_plan", &moe_plan);
+  m.impl("moe_route_plan", &moe_route_plan);
   m.impl("moe_up", &moe_up);
   m.impl("moe_down", &moe_down);
   m.impl("moe_combine", &moe_combine);

@@ -79,23 +79,19 @@ void embed_bigram(Tensor out, const std::optional<Tensor>& cat, bool cat_both, c
 
 int64_t sandwich_join_max_width(bool vec) { return dlia_sandwich_join_max_width(vec ? 1 : 0); }
 
-// y = ya + yb + the token's rows of ey; x += rms(y) wb; out = rms(x) wn, or x itself without wn. Without wb only the second half.
-void sandwich_join(const std::optional<Tensor>& out, Tensor x, OptTensor ya, OptTensor yb, OptTensor ey, OptTensor pair_row, int64_t top,
+// y = ya (as it is, or the sum of its first dimension's partial results) + the token's rows of ey; x += rms(y) wb; out = rms(x) wn, or x itself without wn. Without wb only the second half.
+void sandwich_join(const std::optional<Tensor>& out, Tensor x, OptTensor ya, OptTensor ey, OptTensor pair_row, int64_t top,
                    OptTensor wb, OptTensor wn, double eps) {
   DLIA_ON_DEVICE_OF(x);
   check_fmat(x, "x");
   const int64_t T = x.size(0), H = x.size(1);
-  const float *ap = nullptr, *bp = nullptr, *ep = nullptr; const int* pp = nullptr;
-  long lda = 0, ldb = 0;
+  const float *ap = nullptr, *ep = nullptr; const int* pp = nullptr;
+  long lda = 0, step = 0; int parts = 1;
   if (ya.has_value()) {
-    check_fmat(*ya, "ya");
-    DLIA_CHECK(ya->size(0) >= T && ya->size(1) == H, "sandwich_join: ya [T, H]");
-    ap = ya->data_ptr<float>(); lda = ya->stride(0);
-  }
-  if (yb.has_value()) {
-    check_fmat(*yb, "yb");
-    DLIA_CHECK(yb->size(0) >= T && yb->size(1) == H, "sandwich_join: yb [T, H]");
-    bp = yb->data_ptr<float>(); ldb = yb->stride(0);
+    DLIA_CHECK(ya->is_cuda() && ya->scalar_type() == at::kFloat && (ya->dim() == 2 || ya->dim() == 3) && (ya->size(-1) == 1 || ya->stride(-1) == 1) &&
+               ya->size(-1) == H && ya->size(-2) >= T, "sandwich_join: ya float32 [T, H] or [parts, T, H]");
+    ap = ya->data_ptr<float>(); lda = ya->stride(-2);
+    if (ya->dim() == 3) { parts = (int)ya->size(0); step = ya->stride(0); }
   }
   if (ey.has_value()) {
     check_f32(*ey, "ey");
@@ -104,7 +100,7 @@ void sandwich_join(const std::optional<Tensor>& out, Tensor x, OptTensor ya, Opt
     DLIA_CHECK(pair_row->numel() >= T * top, "sandwich_join: pair_row [T, top]");
     ep = ey->data_ptr<float>(); pp = pair_row->data_ptr<int>();
   }
-  DLIA_CHECK((ap || bp || ep) == wb.has_value(), "sandwich_join: a sublayer's output comes with its norm's weight");
+  DLIA_CHECK((ap || ep) == wb.has_value(), "sandwich_join: a sublayer's output comes with its norm's weight");
   void* op = nullptr; long ldo = 0; int of32 = 1;
   if (out.has_value()) {
     check_act(*out, "out"); check_mat(*out, "out");
@@ -112,7 +108,7 @@ void sandwich_join(const std::optional<Tensor>& out, Tensor x, OptTensor ya, Opt
     op = out->data_ptr(); ldo = out->stride(0); of32 = is_f32(*out);
   }
   DLIA_CHECK(op || wb.has_value(), "sandwich_join: nothing to do");
-  const int rc = dlia_sandwich_join(op, of32, ldo, x.data_ptr<float>(), x.stride(0), ap, lda, bp, ldb, ep, pp, (int)top, opt_f32(wb, H, "wb"),
+  const int rc = dlia_sandwich_join(op, of32, ldo, x.data_ptr<float>(), x.stride(0), ap, lda, parts, step, ep, pp, (int)top, opt_f32(wb, H, "wb"),
                                     opt_f32(wn, H, "wn"), (int)T, (int)H, (float)eps, cur_stream());
   DLIA_CHECK(rc == 0, "sandwich_join: rows of ", H, " are beyond what the kernel holds in registers");
 }
@@ -172,7 +168,7 @@ void relu_act(Tensor act, const Tensor& z, bool glu) {
 TORCH_LIBRARY_FRAGMENT(dlia, m) {
   m.def("embed_bigram(Tensor(a!) out, Tensor(b!)? cat, bool cat_both, Tensor ids, Tensor table, float scale, Tensor? bigram, int mul_prev, int mul_cur, Tensor(c!)? pages, Tensor tok_pos, Tensor tok_seq, Tensor block_table) -> ()");
   m.def("sandwich_join_max_width(bool vec) -> int");
-  m.def("sandwich_join(Tensor(a!)? out, Tensor(b!) x, Tensor? ya, Tensor? yb, Tensor? ey, Tensor? pair_row, int top, Tensor? wb, Tensor? wn, float eps) -> ()");
+  m.def("sandwich_join(Tensor(a!)? out, Tensor(b!) x, Tensor? ya, Tensor? ey, Tensor? pair_row, int top, Tensor? wb, Tensor? wn, float eps) -> ()");
   m.def("qk_prep(Tensor z, int H, int G, int d, int dv, int col_v, Tensor? qw, Tensor? kw, bool unit, float eps, int dims, bool interleaved, Tensor? cos_t, Tensor? sin_t, Tensor(a!) q_out, Tensor(b!) kc, Tensor(c!)? vc, int layout, Tensor tok_pos, Tensor tok_seq, Tensor block_table) -> ()");
   m.def("relu_act(Tensor(a!) act, Tensor z, bool glu) -> ()");
 }

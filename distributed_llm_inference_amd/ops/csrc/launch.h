@@ -175,6 +175,10 @@ void dlia_moe_route(int* sel, float* wts, const float* logits, long ld, int T, i
 void dlia_moe_plan(int* tiles, int* row_tok, int* pair_row, const int* sel, int pairs, int top, int E, int max_rows, int tile_rows,
                    const float* wts, float* row_w, hipStream_t stream);
 // tile_rows: 32 (register-tiled expert kernels, any type and shape) or 128 (LDS-tiled, bf16, K a multiple of 32, aligned rows)
+// both in one call (and for steps of up to 256 tokens in one launch); `experts`: those with rows, E: the router's outputs
+void dlia_moe_route_plan(int* sel, float* wts, const float* logits, long ld, int T, int E, int top, int groups, int keep, float scale,
+                         const float* corr, int softmax, int group_rank, int renorm, int* tiles, int* row_tok, int* pair_row, int experts,
+                         int max_rows, int tile_rows, float* row_w, hipStream_t stream);
 // wg null: experts without a gate, act = relu(x . Wu)^2; row_w: what the rows' inputs are multiplied by
 void dlia_moe_up(void* act, const void* x, const void* wg, const void* wu, int f32, const int* tiles, const int* row_tok,
                  int max_tiles, int wide, int F, int K, long ldx, long lda, float limit, int tile_rows, const float* row_w, hipStream_t stream);
@@ -271,7 +275,8 @@ void dlia_embed_bigram(float* out, void* cat, long ldc, int cat_both, const int*
                        int T, int max_blocks, int num_blocks, int table_rows, int H, int vocab, hipStream_t stream);
 int dlia_sandwich_join_max_width(int vec);
 // Returns 1 (nothing launched) for rows wider than dlia_sandwich_join_max_width.
-int dlia_sandwich_join(void* out, int out_f32, long ldo, float* x, long ldx, const float* ya, long ldya, const float* yb, long ldyb, const float* ey,
+// ya may be `ya_parts` partial sums, `ya_step` floats apart.
+int dlia_sandwich_join(void* out, int out_f32, long ldo, float* x, long ldx, const float* ya, long ldya, int ya_parts, long ya_step, const float* ey,
                        const int* pair_row, int top, const float* wb, const float* wn, int T, int H, float eps, hipStream_t stream);
 // Returns 1 (nothing launched) for types or sizes it does not take.
 int dlia_qk_prep(const void* z, int z_f32, long ldz, int T, int H, int G, int d, int dv, int col_v, const float* qw, const float* kw, int unit,

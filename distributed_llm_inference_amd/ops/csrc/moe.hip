@@ -6,6 +6,7 @@
 //                contiguous blocks of equal size; a block is ranked by its best `group_rank` (1 or 2) choice scores added up;
 //                the `keep` best blocks stay; the `top` best experts of those are chosen (equal scores: the lower index),
 //                weighted score / (sum + 1e-20) * scale, or score * scale without the division.
+//   moe_route_plan   routing and plan together; ONE launch for steps of up to 256 tokens.
 //   moe_plan     one workgroup. Pairs whose choice is not a real expert (an identity expert: index >= E) get row -1 and no
 //                place in a tile. Counts the pairs per expert, lays the experts' row ranges out one after the other, each
 //                padded to whole 32-row tiles, and writes for every padded row its token (or -1), for every pair its row,
@@ -46,12 +47,9 @@ __device__ __forceinline__ float expert_act(float g, float u, float limit) {
 
 __device__ __forceinline__ float relu2(float u) { const float r = fmaxf(u, 0.f); return r * r; }
 
-__global__ __launch_bounds__(64) void moe_route_kernel(int* __restrict__ sel, float* __restrict__ wts,
-                                                       const float* __restrict__ logits, long ld, int T, int E, int top,
-                                                       int groups, int keep, float scale, const float* __restrict__ corr,
-                                                       int softmax, int group_rank, int renorm) {
-  const int t = blockIdx.x * 64 + threadIdx.x;
-  if (t >= T) return;
+__device__ __forceinline__ void route_token(int t, int* __restrict__ sel, float* __restrict__ wts, const float* __restrict__ logits, long ld,
+                                            int E, int top, int groups, int keep, float scale, const float* __restrict__ corr, int softmax,
+                                            int group_rank, int renorm) {
   const float* z = logits + (long)t * ld;
   const int per = E / groups;
   float zmax = 0.f, zinv = 1.f;
@@ -66,7 +64,8 @@ __global__ __launch_bounds__(64) void moe_route_kernel(int* __restrict__ sel, fl
   auto choice = [&](int e) { return corr ? score(e) + corr[e] : score(e); };
   // the groups that stay: `keep` times the best group not yet taken
   unsigned long long gmask[4] = {0ull, 0ull, 0ull, 0ull};
-  for (int r = 0; r < keep; ++r) {
+  if (keep >= groups) gmask[0] = gmask[1] = gmask[2] = gmask[3] = ~0ull;      // (all of them: nothing to rank)
+  for (int r = 0; r < (keep >= groups ? 0 : keep); ++r) {
     int best = -1; float bs = -INFINITY;
     for (int g = 0; g < groups; ++g) {
       if (gmask[g >> 6] >> (g & 63) & 1ull) continue;
@@ -99,6 +98,14 @@ __global__ __launch_bounds__(64) void moe_route_kernel(int* __restrict__ sel, fl
   }
   const float inv = renorm ? scale / (total + 1e-20f) : scale;
   for (int r = 0; r < top; ++r) wts[(long)t * top + r] *= inv;
+}
+
+__global__ __launch_bounds__(64) void moe_route_kernel(int* __restrict__ sel, float* __restrict__ wts,
+                                                       const float* __restrict__ logits, long ld, int T, int E, int top,
+                                                       int groups, int keep, float scale, const float* __restrict__ corr,
+                                                       int softmax, int group_rank, int renorm) {
+  const int t = blockIdx.x * 64 + threadIdx.x;
+  if (t < T) route_token(t, sel, wts, logits, ld, E, top, groups, keep, scale, corr, softmax, group_rank, renorm);
 }
 
 // Lays out the pairs of one layer. expert(i): the expert of pair i (i / top is its token). 1024 threads.
@@ -146,6 +153,21 @@ __global__ __launch_bounds__(1024) void moe_plan_kernel(int* __restrict__ tiles,
   plan_pairs(tiles, row_tok, pair_row, pairs, top, E, max_rows, tile_rows, count, start, fill, &ntiles, [&](int i) { return sel[i]; }, wts, row_w);
 }
 
+// Routing and plan of a step with few tokens in one launch (one workgroup, a thread per token).
+__global__ __launch_bounds__(1024) void moe_route_plan_kernel(int* __restrict__ sel, float* __restrict__ wts, const float* __restrict__ logits,
+                                                              long ld, int T, int E, int top, int groups, int keep, float scale,
+                                                              const float* __restrict__ corr, int softmax, int group_rank, int renorm,
+                                                              int* __restrict__ tiles, int* __restrict__ row_tok, int* __restrict__ pair_row,
+                                                              int experts, int max_rows, int tile_rows, float* __restrict__ row_w) {
+  __shared__ int count[kMoeMaxExperts], start[kMoeMaxExperts], fill[kMoeMaxExperts];
+  __shared__ int ntiles;
+  for (int t = threadIdx.x; t < T; t += 1024) route_token(t, sel, wts, logits, ld, E, top, groups, keep, scale, corr, softmax, group_rank, renorm);
+  __threadfence_block();
+  __syncthreads();
+  plan_pairs(tiles, row_tok, pair_row, T * top, top, experts, max_rows, tile_rows, count, start, fill, &ntiles,
+             [&](int i) { return *(volatile const int*)(sel + i); }, wts, row_w);
+}
+
 constexpr int kPlanDesc = 8;
 constexpr int kTableMaxExperts = 1024;
 
@@ -185,7 +207,16 @@ __global__ __launch_bounds__(256) void glu_act_kernel(OT* __restrict__ act, long
 // and the fragments of the next k-step are on their way while the current ones are multiplied.
 constexpr int kMoeTile = kMoeRows;
 
-template <typename T, typename OT, int NJ, bool GLU>
+// D k-steps of fragments are asked for at once while the D before them are multiplied. FAST: K in whole groups of D steps, aligned
+// rows; then no load is masked (a row without a token reads token 0 or its own stale row, a weight row beyond the last reads row 0:
+// neither reaches a result that is kept), because a load under a mask is a branch and a wait of its own. Else: steps beyond K load zeros.
+template <bool FAST, typename T>
+__device__ __forceinline__ u32x4 step_frag(const T* __restrict__ row, int k, int K, bool valid, int vec_ok) {
+  if constexpr (FAST) return ld16(row + k);
+  else return load_frag<T>(row, k, K, valid, vec_ok);
+}
+
+template <typename T, typename OT, int NJ, bool GLU, int D, bool FAST>
 __global__ __launch_bounds__(256) void moe_up_kernel(OT* __restrict__ act, const T* __restrict__ x, const T* __restrict__ wg,
                                                      const T* __restrict__ wu, const int* __restrict__ tiles,
                                                      const int* __restrict__ row_tok, int F, int K, long ldx, long lda,
@@ -214,31 +245,40 @@ __global__ __launch_bounds__(256) void moe_up_kernel(OT* __restrict__ act, const
   for (int i = 0; i < 2; ++i)
 #pragma unroll
     for (int j = 0; j < NJ; ++j) { ag[i][j] = f32x4{0.f, 0.f, 0.f, 0.f}; au[i][j] = f32x4{0.f, 0.f, 0.f, 0.f}; }
-  u32x4 a[2], g[NJ], u[NJ], an[2], gn[NJ], un[NJ];
-  auto load = [&](u32x4 (&fa)[2], u32x4 (&fg)[NJ], u32x4 (&fu)[NJ], int k0) {
-    const int k = k0 + kq * VEC;
+  struct Frags { u32x4 a[D][2], g[D][GLU ? NJ : 1], u[D][NJ]; };
+  auto load = [&](Frags& f, int k0) {
 #pragma unroll
-    for (int i = 0; i < 2; ++i) fa[i] = load_frag<T>(arow[i], k, K, av[i], vec_ok);
+    for (int s = 0; s < D; ++s) {
+      const int k = k0 + s * KS + kq * VEC;
 #pragma unroll
-    for (int j = 0; j < NJ; ++j) {
-      if constexpr (GLU) fg[j] = load_frag<T>(wg + wrow[j], k, K, wv[j], vec_ok);
-      fu[j] = load_frag<T>(wu + wrow[j], k, K, wv[j], vec_ok);
-    }
-  };
-  load(a, g, u, 0);
-  for (int k0 = 0; k0 < K; k0 += KS) {
-    if (k0 + KS < K) load(an, gn, un, k0 + KS);
-#pragma unroll
-    for (int i = 0; i < 2; ++i)
+      for (int i = 0; i < 2; ++i) f.a[s][i] = step_frag<FAST>(arow[i], k, K, av[i], vec_ok);
 #pragma unroll
       for (int j = 0; j < NJ; ++j) {
-        if constexpr (GLU) ag[i][j] = mma_frag(T{}, a[i], g[j], ag[i][j]);
-        au[i][j] = mma_frag(T{}, a[i], u[j], au[i][j]);
+        if constexpr (GLU) f.g[s][j] = step_frag<FAST>(wg + wrow[j], k, K, wv[j], vec_ok);
+        f.u[s][j] = step_frag<FAST>(wu + wrow[j], k, K, wv[j], vec_ok);
       }
+    }
+  };
+  auto multiply = [&](const Frags& f) {
 #pragma unroll
-    for (int i = 0; i < 2; ++i) a[i] = an[i];
+    for (int s = 0; s < D; ++s)
 #pragma unroll
-    for (int j = 0; j < NJ; ++j) { if constexpr (GLU) g[j] = gn[j]; u[j] = un[j]; }
+      for (int i = 0; i < 2; ++i)
+#pragma unroll
+        for (int j = 0; j < NJ; ++j) {
+          if constexpr (GLU) ag[i][j] = mma_frag(T{}, f.a[s][i], f.g[s][j], ag[i][j]);
+          au[i][j] = mma_frag(T{}, f.a[s][i], f.u[s][j], au[i][j]);
+        }
+  };
+  Frags fa, fb;
+  load(fa, 0);
+  for (int k0 = 0; k0 < K; k0 += 2 * D * KS) {
+    if (k0 + D * KS < K) load(fb, k0 + D * KS);
+    multiply(fa);
+    if (k0 + D * KS < K) {
+      if (k0 + 2 * D * KS < K) load(fa, k0 + 2 * D * KS);
+      multiply(fb);
+    }
   }
 #pragma unroll
   for (int i = 0; i < 2; ++i)
@@ -256,7 +296,7 @@ __global__ __launch_bounds__(256) void moe_up_kernel(OT* __restrict__ act, const
     }
 }
 
-template <typename T, int NJ>
+template <typename T, int NJ, int D, bool FAST>
 __global__ __launch_bounds__(256) void moe_down_kernel(float* __restrict__ y, const T* __restrict__ act, const T* __restrict__ wd,
                                                        const int* __restrict__ tiles, const int* __restrict__ row_tok,
                                                        int H, int F, long lda, int vec_ok) {
@@ -283,25 +323,34 @@ __global__ __launch_bounds__(256) void moe_down_kernel(float* __restrict__ y, co
   for (int i = 0; i < 2; ++i)
 #pragma unroll
     for (int j = 0; j < NJ; ++j) acc[i][j] = f32x4{0.f, 0.f, 0.f, 0.f};
-  u32x4 a[2], w[NJ], an[2], wn[NJ];
-  auto load = [&](u32x4 (&fa)[2], u32x4 (&fw)[NJ], int k0) {
-    const int k = k0 + kq * VEC;
+  struct Frags { u32x4 a[D][2], w[D][NJ]; };
+  auto load = [&](Frags& f, int k0) {
 #pragma unroll
-    for (int i = 0; i < 2; ++i) fa[i] = load_frag<T>(arow[i], k, F, av[i], vec_ok);
+    for (int s = 0; s < D; ++s) {
+      const int k = k0 + s * KS + kq * VEC;
 #pragma unroll
-    for (int j = 0; j < NJ; ++j) fw[j] = load_frag<T>(wrow[j], k, F, wv[j], vec_ok);
+      for (int i = 0; i < 2; ++i) f.a[s][i] = step_frag<FAST>(arow[i], k, F, av[i], vec_ok);
+#pragma unroll
+      for (int j = 0; j < NJ; ++j) f.w[s][j] = step_frag<FAST>(wrow[j], k, F, wv[j], vec_ok);
+    }
   };
-  load(a, w, 0);
-  for (int k0 = 0; k0 < F; k0 += KS) {
-    if (k0 + KS < F) load(an, wn, k0 + KS);
+  auto multiply = [&](const Frags& f) {
 #pragma unroll
-    for (int i = 0; i < 2; ++i)
+    for (int s = 0; s < D; ++s)
 #pragma unroll
-      for (int j = 0; j < NJ; ++j) acc[i][j] = mma_frag(T{}, a[i], w[j], acc[i][j]);
+      for (int i = 0; i < 2; ++i)
 #pragma unroll
-    for (int i = 0; i < 2; ++i) a[i] = an[i];
-#pragma unroll
-    for (int j = 0; j < NJ; ++j) w[j] = wn[j];
+        for (int j = 0; j < NJ; ++j) acc[i][j] = mma_frag(T{}, f.a[s][i], f.w[s][j], acc[i][j]);
+  };
+  Frags fa, fb;
+  load(fa, 0);
+  for (int k0 = 0; k0 < F; k0 += 2 * D * KS) {
+    if (k0 + D * KS < F) load(fb, k0 + D * KS);
+    multiply(fa);
+    if (k0 + D * KS < F) {
+      if (k0 + 2 * D * KS < F) load(fa, k0 + 2 * D * KS);
+      multiply(fb);
+    }
   }
 #pragma unroll
   for (int i = 0; i < 2; ++i)
@@ -316,16 +365,17 @@ __global__ __launch_bounds__(256) void moe_down_kernel(float* __restrict__ y, co
 
 // Steps with many rows (prompts): 128-row tiles, operands staged through LDS. A workgroup owns one row tile by 128 weight rows —
 // for the up projection 64 gate rows and the 64 up rows of the same columns, so the activation is formed in registers; for the
-// down projection 128 output columns — and walks K in steps of 32: every thread brings four 16-byte pieces of the next step
-// (two of the rows, gathered through the plan for the up projection; two of the weights) into registers while the current
-// step is multiplied, then parks them in the other half of a double buffer. Rows are 80 bytes apart in LDS, which spreads the
+// down projection 128 output columns — and walks K in steps of 32: every thread keeps four 16-byte pieces of each of the next
+// kBigAhead steps (two of the rows, gathered through the plan for the up projection; two of the weights) on their way into
+// registers while the current step is multiplied, and parks the next step's in the other half of a double buffer. Rows are 80 bytes apart in LDS, which spreads the
 // fragment reads of a 16-row tile over the banks. A wave multiplies 32 rows by all 128 weight rows: 10 fragment reads for 16
 // MFMAs. bf16, K a multiple of 32 with 16-byte aligned rows (the caller falls back to the register-tiled kernels otherwise).
+constexpr int kBigAhead = 2;            // steps on their way at once (one: a step costs a memory latency; three: too many registers)
 constexpr int kBigStride = 40;          // bf16 elements between rows in LDS (64 bytes of data + 16 of padding)
 
 // KIND 0: down; 1: gate and up; 2: up alone (128 columns per workgroup, the square of relu).
 template <int KIND>
-__global__ __launch_bounds__(256) void moe_big_kernel(bf16* __restrict__ act_out, float* __restrict__ y_out, const bf16* __restrict__ a,
+__global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(3))) void moe_big_kernel(bf16* __restrict__ act_out, float* __restrict__ y_out, const bf16* __restrict__ a,
                                                       const bf16* __restrict__ w0, const bf16* __restrict__ w1,
                                                       const int* __restrict__ tiles, const int* __restrict__ row_tok, int N, int K,
                                                       long lda, long ldo, float limit, const float* __restrict__ row_w) {
@@ -337,43 +387,46 @@ __global__ __launch_bounds__(256) void moe_big_kernel(bf16* __restrict__ act_out
   const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, r16 = lane & 15, kq = lane >> 4;
   const int n0 = blockIdx.x * (GLU ? 64 : 128);                 // first output column of the workgroup
   // the four pieces this thread stages per k-step: pieces 2 tid, 2 tid + 1 of the 512 row pieces, and of the 512 weight pieces
-  const bf16* src[4]; bool ok[4]; int dst[4];
+  // (nothing is masked: a row without a token reads token 0 or its own stale row, a weight row beyond N reads row 0, and neither
+  // reaches a result that is kept; loads under a mask would each be a branch and a wait of its own)
+  const bf16* src[4]; int dst[4];
 #pragma unroll
   for (int i = 0; i < 2; ++i) {
     const int c = tid * 2 + i, row = c >> 2, part = c & 3;
     const int grow = tile * kMoeBigRows + row;
-    if constexpr (UP) { const int tok = row_tok[grow]; ok[i] = tok >= 0; src[i] = a + (long)(ok[i] ? tok : 0) * lda + part * 8; }
-    else { ok[i] = row_tok[grow] >= 0; src[i] = a + (long)grow * lda + part * 8; }
+    if constexpr (UP) { const int tok = row_tok[grow]; src[i] = a + (long)(tok >= 0 ? tok : 0) * lda + part * 8; }
+    else src[i] = a + (long)grow * lda + part * 8;
     dst[i] = row * kBigStride + part * 8;
     // weights: LDS rows 128 .. 255
     int wr; const bf16* base;
     if constexpr (GLU) { wr = n0 + (row & 63); base = row < 64 ? w0 : w1; }
     else { wr = n0 + row; base = w0; }
-    ok[2 + i] = wr < N;
-    src[2 + i] = base + ((long)e * N + (ok[2 + i] ? wr : 0)) * K + part * 8;
+    src[2 + i] = base + ((long)e * N + (wr < N ? wr : 0)) * K + part * 8;
     dst[2 + i] = (128 + row) * kBigStride + part * 8;
   }
-  u32x4 st[4];
-  auto fetch = [&](int k0) {
+  u32x4 st[kBigAhead][4];               // step s waits in st[s % kBigAhead]
+  const int steps = K / 32;
+  auto fetch = [&](u32x4 (&v)[4], int s) {
+    const int k0 = (s < steps ? s : steps - 1) * 32;             // (beyond the end: the last step once more, never used)
 #pragma unroll
-    for (int i = 0; i < 4; ++i) st[i] = ok[i] ? ld16(src[i] + k0) : u32x4{0u, 0u, 0u, 0u};
+    for (int i = 0; i < 4; ++i) v[i] = ld16(src[i] + k0);
   };
-  auto park = [&](int buf) {
+  auto park = [&](int buf, const u32x4 (&v)[4]) {
 #pragma unroll
-    for (int i = 0; i < 4; ++i) *reinterpret_cast<u32x4*>(&lds[buf][dst[i]]) = st[i];
+    for (int i = 0; i < 4; ++i) *reinterpret_cast<u32x4*>(&lds[buf][dst[i]]) = v[i];
   };
   f32x4 acc[2][8];
 #pragma unroll
   for (int i = 0; i < 2; ++i)
 #pragma unroll
     for (int j = 0; j < 8; ++j) acc[i][j] = f32x4{0.f, 0.f, 0.f, 0.f};
-  fetch(0);
-  park(0);
+#pragma unroll
+  for (int s = 0; s < kBigAhead; ++s) fetch(st[s], s);
+  park(0, st[0]);
+  fetch(st[0], kBigAhead);
   __syncthreads();
-  int buf = 0;
-  for (int k0 = 0; k0 < K; k0 += 32) {
-    const bool more = k0 + 32 < K;
-    if (more) fetch(k0 + 32);
+  auto step = [&](int s, u32x4 (&next)[4]) {
+    const int buf = s & 1;
     u32x4 fa[2], fw[8];
 #pragma unroll
     for (int i = 0; i < 2; ++i) fa[i] = *reinterpret_cast<const u32x4*>(&lds[buf][(wave * 32 + i * 16 + r16) * kBigStride + kq * 8]);
@@ -383,10 +436,14 @@ __global__ __launch_bounds__(256) void moe_big_kernel(bf16* __restrict__ act_out
     for (int i = 0; i < 2; ++i)
 #pragma unroll
       for (int j = 0; j < 8; ++j) acc[i][j] = mfma16(fa[i], fw[j], acc[i][j]);
-    if (more) park(buf ^ 1);
+    park(buf ^ 1, next);
+    fetch(next, s + 1 + kBigAhead);
     __syncthreads();
-    buf ^= 1;
-  }
+  };
+  static_assert(kBigAhead == 2, "the walk below takes steps in pairs");
+  int s = 0;
+  for (; s + 2 <= steps; s += 2) { step(s, st[1]); step(s + 1, st[0]); }
+  if (s < steps) step(s, st[1]);
 #pragma unroll
   for (int i = 0; i < 2; ++i)
 #pragma unroll
@@ -446,23 +503,42 @@ extern "C" void dlia_moe_plan(int* tiles, int* row_tok, int* pair_row, const int
                      tile_rows, wts, row_w);
 }
 
+extern "C" void dlia_moe_route_plan(int* sel, float* wts, const float* logits, long ld, int T, int E, int top, int groups, int keep, float scale,
+                                    const float* corr, int softmax, int group_rank, int renorm, int* tiles, int* row_tok, int* pair_row,
+                                    int experts, int max_rows, int tile_rows, float* row_w, hipStream_t stream) {
+  if (T <= 0) return;
+  if (T <= 256) {
+    hipLaunchKernelGGL(dlia::moe_route_plan_kernel, dim3(1), dim3(1024), 0, stream, sel, wts, logits, ld, T, E, top, groups, keep, scale, corr,
+                       softmax, group_rank, renorm, tiles, row_tok, pair_row, experts, max_rows, tile_rows, row_w);
+    return;
+  }
+  dlia_moe_route(sel, wts, logits, ld, T, E, top, groups, keep, scale, corr, softmax, group_rank, renorm, stream);
+  dlia_moe_plan(tiles, row_tok, pair_row, sel, T * top, top, experts, max_rows, tile_rows, wts, row_w, stream);
+}
+
 // Steps with few rows (decoding) take narrow column blocks: more workgroups stream the experts' weights at once.
 template <typename T, typename OT, int NJ>
 static void launch_moe_up(void* act, const void* x, const void* wg, const void* wu, const int* tiles, const int* row_tok, int max_tiles,
                           int F, int K, long ldx, long lda, float limit, int ok, const float* row_w, hipStream_t stream) {
   const dim3 grid((F + 64 * NJ - 1) / (64 * NJ), max_tiles);
-  if (wg)
-    hipLaunchKernelGGL((dlia::moe_up_kernel<T, OT, NJ, true>), grid, dim3(256), 0, stream, (OT*)act, (const T*)x, (const T*)wg, (const T*)wu,
-                       tiles, row_tok, F, K, ldx, lda, limit, ok, row_w);
-  else
-    hipLaunchKernelGGL((dlia::moe_up_kernel<T, OT, NJ, false>), grid, dim3(256), 0, stream, (OT*)act, (const T*)x, (const T*)wg, (const T*)wu,
-                       tiles, row_tok, F, K, ldx, lda, limit, ok, row_w);
+  constexpr int D = NJ == 1 ? 4 : 1;
+  const bool fast = ok && K % (D * 64 / (int)sizeof(T)) == 0;
+#define DLIA_UP(GLU, FAST)                                                                                                                 \
+  hipLaunchKernelGGL((dlia::moe_up_kernel<T, OT, NJ, GLU, D, FAST>), grid, dim3(256), 0, stream, (OT*)act, (const T*)x, (const T*)wg, (const T*)wu, \
+                     tiles, row_tok, F, K, ldx, lda, limit, ok, row_w)
+  if (wg) { if (fast) DLIA_UP(true, true); else DLIA_UP(true, false); }
+  else { if (fast) DLIA_UP(false, true); else DLIA_UP(false, false); }
+#undef DLIA_UP
 }
 template <typename T, int NJ>
 static void launch_moe_down(float* y, const void* act, const void* wd, const int* tiles, const int* row_tok, int max_tiles, int H, int F,
                             long lda, int ok, hipStream_t stream) {
   const dim3 grid((H + 64 * NJ - 1) / (64 * NJ), max_tiles);
-  hipLaunchKernelGGL((dlia::moe_down_kernel<T, NJ>), grid, dim3(256), 0, stream, y, (const T*)act, (const T*)wd, tiles, row_tok, H, F, lda, ok);
+  constexpr int D = NJ == 1 ? 4 : 1;
+  if (ok && F % (D * 64 / (int)sizeof(T)) == 0)
+    hipLaunchKernelGGL((dlia::moe_down_kernel<T, NJ, D, true>), grid, dim3(256), 0, stream, y, (const T*)act, (const T*)wd, tiles, row_tok, H, F, lda, ok);
+  else
+    hipLaunchKernelGGL((dlia::moe_down_kernel<T, NJ, D, false>), grid, dim3(256), 0, stream, y, (const T*)act, (const T*)wd, tiles, row_tok, H, F, lda, ok);
 }
 
 extern "C" void dlia_moe_up(void* act, const void* x, const void* wg, const void* wu, int f32, const int* tiles, const int* row_tok,

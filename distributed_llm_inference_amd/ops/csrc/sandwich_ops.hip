@@ -7,8 +7,8 @@
 //                  the rows the pass map reads. The previous token of a portion's first token comes from the sequence's cache
 //                  blocks: every token's id is written to its place in a page of 32 ids per block, the way keys and values are,
 //                  so it needs no slot state, moves with the block table, and a step that is run twice writes the same.
-//   sandwich_join  one launch per sublayer boundary: the finished sublayer's output (a GEMM's, plus a shared expert's, plus the
-//                  token's routed expert rows) is RMS-normed over the row, weighted (the residual multiplier rides in the
+//   sandwich_join  one launch per sublayer boundary: the finished sublayer's output (a GEMM's, whole or as the partial sums of its
+//                  key splits, plus the token's routed expert rows) is RMS-normed over the row, weighted (the residual multiplier rides in the
 //                  weight) and added to the stream; the next sublayer's normed input leaves in the GEMMs' type, or the stream
 //                  itself does (the other half of the pass map's rows). A row stays in registers from its load to its store.
 //   qk_prep        between an attention mixer's input projection and its cache: per head RMS norm of q and k with a weight ahead of
@@ -76,8 +76,8 @@ __global__ __launch_bounds__(kSandThreads) void embed_bigram_kernel(
 // ---- sublayer boundary -----------------------------------------------------------------------------------------------
 template <typename OT, int V, int NR>
 __global__ __launch_bounds__(kSandThreads) void sandwich_join_kernel(
-    OT* __restrict__ out, long ldo, float* __restrict__ x, long ldx, const float* __restrict__ ya, long ldya, const float* __restrict__ yb,
-    long ldyb, const float* __restrict__ ey, const int* __restrict__ pair_row, int top, const float* __restrict__ wb,
+    OT* __restrict__ out, long ldo, float* __restrict__ x, long ldx, const float* __restrict__ ya, long ldya, int ya_parts, long ya_step,
+    const float* __restrict__ ey, const int* __restrict__ pair_row, int top, const float* __restrict__ wb,
     const float* __restrict__ wn, int H, float eps) {
   __shared__ float scratch[16];
   const int t = blockIdx.x, units = H / V, nt = blockDim.x;
@@ -96,11 +96,16 @@ __global__ __launch_bounds__(kSandThreads) void sandwich_join_kernel(
       const int u = threadIdx.x + k * nt;
       if (u >= units) break;
       const int c = u * V;
-      if (ya) {
-        y[k] = ldu<V>(ya + (long)t * ldya + c);
-      } else {
 #pragma unroll
-        for (int e = 0; e < V; ++e) y[k].v[e] = 0.f;
+      for (int e = 0; e < V; ++e) y[k].v[e] = 0.f;
+      if (ya) {
+        const float* yr = ya + (long)t * ldya + c;
+#pragma unroll 4
+        for (int i = 0; i < ya_parts; ++i) {
+          const Unit<V> a = ldu<V>(yr + i * ya_step);
+#pragma unroll
+          for (int e = 0; e < V; ++e) y[k].v[e] += a.v[e];
+        }
       }
       if (ey)
         for (int i = 0; i < top; ++i) {
@@ -110,11 +115,6 @@ __global__ __launch_bounds__(kSandThreads) void sandwich_join_kernel(
 #pragma unroll
           for (int e = 0; e < V; ++e) y[k].v[e] += a.v[e];
         }
-      if (yb) {
-        const Unit<V> a = ldu<V>(yb + (long)t * ldyb + c);
-#pragma unroll
-        for (int e = 0; e < V; ++e) y[k].v[e] += a.v[e];
-      }
 #pragma unroll
       for (int e = 0; e < V; ++e) ss += y[k].v[e] * y[k].v[e];
     }
@@ -164,6 +164,7 @@ struct PrepParams {
   int T, H, G, d, dv, col_v;            // col_v < 0: the values are the keys as projected
   const float *qw, *kw; int unit; float eps;
   int dims, interleaved; const float *cos_t, *sin_t; int table_pos;
+  int whole;                            // rotated parts come in whole runs of V entries: vector reads of partners and angles
   void* q_out; long ldqo;
   void* kc; void* vc; int layout;       // 0: rows of k and of v; 1: values key-contiguous; 2: the fragment-ordered slabs (kv_layout.h)
   const int *tok_pos, *tok_seq, *block_table; int max_blocks, num_blocks, table_rows;
@@ -269,7 +270,7 @@ __global__ __launch_bounds__(kSandThreads) void qk_prep_kernel(PrepParams p) {
 #pragma unroll
     for (int c = 0; c < NCH; ++c) {
       const int i = (c * LPH + l) * V;
-      if (!is_v && i < p.d) store_vals<float, V>(row + i, f[c]);
+      if (!is_v && i < p.d && !(p.whole && p.interleaved)) store_vals<float, V>(row + i, f[c]);
     }
     __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
     __builtin_amdgcn_wave_barrier();
@@ -279,10 +280,35 @@ __global__ __launch_bounds__(kSandThreads) void qk_prep_kernel(PrepParams p) {
       const float* cs = p.cos_t + (long)pos * half;
       const float* sn = p.sin_t + (long)pos * half;
 #pragma unroll
-      for (int c = 0; c < NCH; ++c)
+      for (int c = 0; c < NCH; ++c) {
+        const int i0 = (c * LPH + l) * V;
+        if constexpr (V == 8) {
+          if (p.whole) {
+            if (i0 >= p.dims) break;
+            if (p.interleaved) {                    // four pairs of this lane's own
+              const f32x4 cv = *reinterpret_cast<const f32x4*>(cs + (i0 >> 1)), sv = *reinterpret_cast<const f32x4*>(sn + (i0 >> 1));
+#pragma unroll
+              for (int e = 0; e < 4; ++e) {
+                const float u = f[c][2 * e], v = f[c][2 * e + 1];
+                f[c][2 * e] = u * cv[e] - v * sv[e];
+                f[c][2 * e + 1] = v * cv[e] + u * sv[e];
+              }
+            } else {                                // eight entries against the partner run of the other half
+              const bool first = i0 < half;
+              const int pi = first ? i0 : i0 - half;
+              float o[8], cv[8], sv[8];
+              load_vals<float, 8>(row + (first ? i0 + half : pi), o);
+              load_vals<float, 8>(cs + pi, cv);
+              load_vals<float, 8>(sn + pi, sv);
+#pragma unroll
+              for (int e = 0; e < 8; ++e) f[c][e] = f[c][e] * cv[e] + (first ? -o[e] : o[e]) * sv[e];
+            }
+            continue;
+          }
+        }
 #pragma unroll
         for (int e = 0; e < V; ++e) {
-          const int i = (c * LPH + l) * V + e;
+          const int i = i0 + e;
           if (i < p.dims) {
             const bool first = p.interleaved ? !(i & 1) : i < half;
             const int pi = p.interleaved ? i >> 1 : (first ? i : i - half);
@@ -290,6 +316,7 @@ __global__ __launch_bounds__(kSandThreads) void qk_prep_kernel(PrepParams p) {
             f[c][e] = f[c][e] * cs[pi] + (first ? -other : other) * sn[pi];
           }
         }
+      }
     }
   }
   if (p.unit && !is_v) {
@@ -355,19 +382,19 @@ extern "C" void dlia_embed_bigram(float* out, void* cat, long ldc, int cat_both,
 
 extern "C" int dlia_sandwich_join_max_width(int vec) { return vec ? kSandThreads * 4 * 16 : kSandThreads * 32; }
 
-extern "C" int dlia_sandwich_join(void* out, int out_f32, long ldo, float* x, long ldx, const float* ya, long ldya, const float* yb,
-                                  long ldyb, const float* ey, const int* pair_row, int top, const float* wb, const float* wn, int T, int H,
+extern "C" int dlia_sandwich_join(void* out, int out_f32, long ldo, float* x, long ldx, const float* ya, long ldya, int ya_parts,
+                                  long ya_step, const float* ey, const int* pair_row, int top, const float* wb, const float* wn, int T, int H,
                                   float eps, hipStream_t stream) {
   if (T <= 0) return 0;
   auto al = [](const void* p) { return (uintptr_t)p % 16 == 0; };
-  const bool vec = H % 4 == 0 && ldx % 4 == 0 && ldo % 4 == 0 && ldya % 4 == 0 && ldyb % 4 == 0 && al(x) && al(out) && al(ya) && al(yb) &&
+  const bool vec = H % 4 == 0 && ldx % 4 == 0 && ldo % 4 == 0 && ldya % 4 == 0 && ya_step % 4 == 0 && al(x) && al(out) && al(ya) &&
                    al(ey) && al(wb) && al(wn);
   if (H > dlia_sandwich_join_max_width(vec)) return 1;
   const int units = vec ? H / 4 : H;
   const int threads = units <= 64 ? 64 : units <= 128 ? 128 : kSandThreads;
   const int nr = (units + threads - 1) / threads;
 #define DLIA_JOIN_OT(OT, V, NR)                                                                                                   \
-  hipLaunchKernelGGL((sandwich_join_kernel<OT, V, NR>), dim3(T), dim3(threads), 0, stream, (OT*)out, ldo, x, ldx, ya, ldya, yb, ldyb, ey, \
+  hipLaunchKernelGGL((sandwich_join_kernel<OT, V, NR>), dim3(T), dim3(threads), 0, stream, (OT*)out, ldo, x, ldx, ya, ldya, ya_parts, ya_step, ey, \
                      pair_row, top, wb, wn, H, eps)
 #define DLIA_JOIN(V, NR)                                                                            \
   do { if (out_f32) DLIA_JOIN_OT(float, V, NR); else DLIA_JOIN_OT(bf16, V, NR); } while (0)
@@ -383,13 +410,14 @@ extern "C" int dlia_sandwich_join(void* out, int out_f32, long ldo, float* x, lo
 }
 
 template <typename ZT, typename QT, typename CT>
-static int launch_prep(const PrepParams& p, hipStream_t stream) {
+static int launch_prep(PrepParams p, hipStream_t stream) {
   auto al = [](const void* q) { return (uintptr_t)q % 16 == 0; };
   const int widest = p.d > p.dv ? p.d : p.dv;
   const long items = (long)p.T * (p.H + p.G + (p.col_v >= 0 ? p.G : 0));
   const bool vec = p.d % 8 == 0 && p.dv % 8 == 0 && p.ldz % 8 == 0 && p.ldqo % 8 == 0 && (p.col_v < 0 || p.col_v % 8 == 0) && al(p.z) &&
                    al(p.q_out) && al(p.kc) && al(p.vc);
   if (widest > 512 || (p.layout == 2 && !(vec && sizeof(CT) == 2 && p.d == p.dv && (p.d == 64 || p.d == 128)))) return 1;
+  p.whole = vec && p.dims % (p.interleaved ? 8 : 16) == 0 && al(p.cos_t) && al(p.sin_t);
   const size_t row = ((p.d + 3) / 4 * 4 + 4) * sizeof(float);
 #define DLIA_PREP(V, LPH, NCH)                                                                                                    \
   hipLaunchKernelGGL((qk_prep_kernel<ZT, QT, CT, V, LPH, NCH>), dim3((unsigned)((items + kSandThreads / LPH - 1) / (kSandThreads / LPH))),  \
@@ -408,7 +436,7 @@ extern "C" int dlia_qk_prep(const void* z, int z_f32, long ldz, int T, int H, in
                             int q_f32, long ldqo, void* kc, void* vc, int cache_f32, int layout, const int* tok_pos, const int* tok_seq,
                             const int* block_table, int max_blocks, int num_blocks, int table_rows, hipStream_t stream) {
   if (T <= 0) return 0;
-  const PrepParams p{z, ldz, T, H, G, d, dv, col_v, qw, kw, unit, eps, dims, interleaved, cos_t, sin_t, table_pos, q_out, ldqo, kc, vc, layout,
+  const PrepParams p{z, ldz, T, H, G, d, dv, col_v, qw, kw, unit, eps, dims, interleaved, cos_t, sin_t, table_pos, 0, q_out, ldqo, kc, vc, layout,
                      tok_pos, tok_seq, block_table, max_blocks, num_blocks, table_rows};
   if (cache_f32) return z_f32 && q_f32 ? launch_prep<float, float, float>(p, stream) : 1;
   if (z_f32) return q_f32 ? launch_prep<float, float, bf16>(p, stream) : launch_prep<float, bf16, bf16>(p, stream);

@@ -125,7 +125,7 @@ def test_embedding_hip(dtype, H, buckets, mp, mc):
 @pytest.mark.parametrize("H", [37, 48, 200, 1036, 2048, 3001, 8192])
 @pytest.mark.parametrize("out_dtype", [torch.float32, torch.bfloat16])
 def test_boundary_hip(H, out_dtype):
-    """Every use of the boundary kernel: a GEMM's output alone, with a shared expert's and routed rows in any order, before a norm, before
+    """Every use of the boundary kernel: a GEMM's output whole or in partial sums, alone and with routed rows in any order, before a norm, before
     the pass map (the stream itself, into half of wider rows), at the end, and the norm alone."""
     K, dev, T, eps, top = _K(), "cuda", 9, 1e-5, 2
     f = lambda t: t.float().to(dev).contiguous()
@@ -140,12 +140,14 @@ def test_boundary_hip(H, out_dtype):
     E2 = E.clone()
     E2[1, 1] = 0.0
     tol = 2e-5 if out_dtype == torch.float32 else 1e-2
-    for a, b, e in ((ya, None, None), (None, yb, E2), (None, None, E2), (ya, yb, None)):
-        y = sum(t for t in (a, b, e.sum(1) if e is not None else None) if t is not None)
+    parts = torch.zeros(5, T + 2, H + 4, device=dev)
+    parts[:, :T, :H] = f(torch.stack([rnd(T, H, seed=20 + i) for i in range(5)]))
+    psum = sum(rnd(T, H, seed=20 + i) for i in range(5))
+    pad[:, :H] = f(ya)
+    for a, given, e in ((ya, pad[:, :H], None), (yb, f(yb), E2), (None, None, E2), (psum, parts[:, :, :H], None), (psum, parts[:, :, :H], E2)):
+        y = sum(t for t in (a, e.sum(1) if e is not None else None) if t is not None)
         want = x + O.rms(y, eps, wb)
-        if a is not None:
-            pad[:, :H] = f(a)
-        args = (pad[:, :H] if a is not None else None, f(b) if b is not None else None, ey if e is not None else None, pairs if e is not None else None, top, f(wb))
+        args = (given, ey if e is not None else None, pairs if e is not None else None, top, f(wb))
         h, out = f(x), torch.zeros(T, H, device=dev, dtype=out_dtype)
         K.sandwich_join(out, h, *args, f(wn), eps)
         close(h, want)
@@ -159,7 +161,7 @@ def test_boundary_hip(H, out_dtype):
         K.sandwich_join(None, h, *args, None, eps)
         close(h, want)
     h, out = f(x), torch.zeros(T, H, device=dev, dtype=out_dtype)
-    K.sandwich_join(out, h, None, None, None, None, 1, None, f(wn), eps)
+    K.sandwich_join(out, h, None, None, None, 1, None, f(wn), eps)
     close(out, O.rms(x, eps, wn), tol)
     assert torch.equal(h, f(x))
 
@@ -203,6 +205,13 @@ def test_routed_feed_forward_hip(dtype, H, ff, experts, top, T):
     tiles, row_tok, pair_row = (torch.full((n,), 77777, dtype=torch.int32, device=dev) for n in (1 + nt, tr * nt, T * top))
     row_w = torch.full((tr * nt,), float("nan"), device=dev)
     K.moe_plan(tiles, row_tok, pair_row, sel, T * top, top, experts, tr, wts, row_w)
+    # both in one call: the same choices and weights, every pair in a row of its own in a tile of its expert
+    again = [torch.full_like(t, 7) for t in (sel, wts, tiles, row_tok, pair_row, row_w)]
+    K.moe_route_plan(again[0], again[1], z, top, 1, 1, 1.0, None, False, 1, False, again[2], again[3], again[4], experts, tr, again[5])
+    assert torch.equal(again[0], sel) and torch.equal(again[1], wts) and torch.equal(again[2][:1 + int(tiles[0])], tiles[:1 + int(tiles[0])])
+    pr = again[4].cpu().long()
+    assert pr.unique().numel() == T * top and torch.equal(again[2].cpu()[1 + pr // tr], sel.cpu()) and torch.equal(again[5].cpu()[pr], wts.cpu())
+    assert torch.equal(again[3].cpu()[pr], torch.arange(T * top, dtype=torch.int32) // top)
     pr = pair_row.cpu().long()
     assert pr.unique().numel() == T * top and torch.equal(row_w.cpu()[pr], wts.cpu())
     eact, ey = torch.full((tr * nt, ff), 3.0, device=dev, dtype=dtype), torch.full((tr * nt, H), 3.0, device=dev)
@@ -213,7 +222,7 @@ def test_routed_feed_forward_hip(dtype, H, ff, experts, top, T):
     K.relu_act(act, f(x @ P["shared.up"].T), False)
     yb = (act.float() @ P["shared.down"].float().to(dev).T).contiguous()
     h = torch.zeros(T, H, device=dev)
-    K.sandwich_join(None, h, None, yb, ey, pair_row, top, torch.ones(H, device=dev), None, eps)
+    K.sandwich_join(None, h, yb, ey, pair_row, top, torch.ones(H, device=dev), None, eps)
     close(h, O.rms(ref, eps), 3e-5 if dtype == torch.float32 else 2e-2)
 
 
